@@ -17,6 +17,11 @@
 //                     (output [T][H][G dv]: what mixing the heads' weight maps after the softmax needs),
 //                     c >= 0 head c's for every query head.
 //                     `gate_elem`: the gate has one logit per output entry, out[t][h][d] *= sigmoid(gate[t][h dv + d]).
+//                     softcap > 0: the scaled score is bounded, score <- softcap tanh(score / softcap), before the
+//                     distance penalty. keep > 0 (sliding windows): the sequence's first `keep` keys stay visible
+//                     (j < keep and j <= i) besides the window. The keys a query can see are then walked in order
+//                     through a numbering without the gap: 0 .. kept - 1 are the kept keys before the window's first
+//                     one, kept, kept + 1, .. the window's, so that a handful of kept keys share a tile with the window.
 //                     `wfn` = kWeightsSigmoid: no softmax; the weight of a visible key is sigmoid(score + hbias[h]),
 //                     not normalised over the keys (no sink).
 //   talk_mix          out[t][h] = sigmoid(gate[t][h]) * sum_g talk[h][g] * o_all[t][g][c(h)], c(h) = h / (H / G)
@@ -32,6 +37,10 @@ namespace xgm {
 constexpr int kMaskCausal = 0, kMaskWindow = 1, kMaskChunk = 2;
 constexpr int kValuesOwn = -1, kValuesAll = -2;
 constexpr int kWeightsSoftmax = 0, kWeightsSigmoid = 1;
+// matrix-core forms of the bounded softmax: kWeightsBounded needs no running maximum (|score| <= softcap, so every
+// exponential and every sum of them stays in range without a reference), kWeightsCapped keeps one (large bounds, sinks)
+constexpr int kWeightsBounded = 2, kWeightsCapped = 3;
+constexpr float kBoundedMaxLog2 = 90.f;   // largest bound in units of ln 2: 2^90 x 2^20 keys x values stays far from 2^127
 
 __device__ __forceinline__ int first_visible(int mask, int size, int pos) {
   if (mask == kMaskWindow) return max(0, pos - size + 1);
@@ -87,7 +96,7 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
     const int32_t* __restrict__ token_seq, const float* __restrict__ temp, const float* __restrict__ sink,
     T* __restrict__ out, int H, int G, int dk, int dv_head, int mask, int size, float scale, int KT,
     const T* __restrict__ gate, int64_t ld_gate, const float* __restrict__ r1, const float* __restrict__ r2, int vmode,
-    int gate_elem, int wfn, const float* __restrict__ hbias) {
+    int gate_elem, int wfn, const float* __restrict__ hbias, float softcap, int keep) {
   extern __shared__ float smem[];
   // dv: value columns per query head; voff: where they start in a cached row of G * dv_head values
   const int dv = vmode == kValuesAll ? G * dv_head : dv_head;
@@ -131,11 +140,12 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
   const int LPK = 64 / KT;  // lanes per key in the score phase
   const int kj = lane / LPK, part = lane % LPK;
   const int32_t* bt = block_tables + (int64_t)s * bt_width;
-  for (int k0 = j0; k0 <= pos; k0 += KT) {
-    const int n = min(KT, pos - k0 + 1);
+  const int kept = min(keep, j0), gap = j0 - kept, nkeys = pos + 1 - gap;   // key v of the walk: v, or v + gap from `kept` on
+  for (int k0 = 0; k0 < nkeys; k0 += KT) {
+    const int n = min(KT, nkeys - k0);
     __syncthreads();  // the previous tile is consumed (and qs is written, on the first pass)
     for (int jj = wave; jj < n; jj += 4) {
-      const int key = k0 + jj;
+      const int key = k0 + jj < kept ? k0 + jj : k0 + jj + gap;
       const int64_t row = (int64_t)bt[key / bs] * bs + key % bs;
       const T* ks = kcache + (row * G + g) * dk;
       const T* vs = vcache + row * G * dv_head + voff;
@@ -153,7 +163,8 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
         for (int d = part; d < dk; d += LPK) sc += qh[d] * kr[d];
       }
       for (int o = 1; o < LPK; o <<= 1) sc += __shfl_xor(sc, o, 64);
-      if (r1 && kj < n) sc -= pen1[a] * log1pf(pen2[a] * (float)(pos - (k0 + kj)));
+      if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+      if (r1 && kj < n) sc -= pen1[a] * log1pf(pen2[a] * (float)(pos - (k0 + kj < kept ? k0 + kj : k0 + kj + gap)));
       float p;
       if (wfn == kWeightsSigmoid) {   // every visible key weighs sigmoid(score + bias), whatever the others do
         p = kj < n ? sigmoidf(sc + hb[a]) : 0.f;
@@ -228,7 +239,7 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
     const float* __restrict__ sink, bf16* __restrict__ out, int H, int G, int dk, int dv_head, int mask, int size,
     float scale, int RH, int head_slots, float* __restrict__ part_o, float* __restrict__ part_ml, int Ttot,
     const bf16* __restrict__ gate, int64_t ld_gate, const float* __restrict__ r1, const float* __restrict__ r2, int vmode,
-    int gate_elem, const float* __restrict__ hbias) {
+    int gate_elem, const float* __restrict__ hbias, float softcap, int keep) {
   extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
   // dv: value columns per query head; voff: where they start in a cached row of G * dv_head values
   const int dv = vmode == kValuesAll ? G * dv_head : dv_head;
@@ -269,9 +280,12 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
   const int pos_w0 = ctx + min(tw, qn - 1);
   const int lo_w1 = first_visible(mask, size, ctx + min(head_slots ? 0 : tw + 15, qn - 1));
   const int nkk = dk / 32, nmt = dv / 16;
-  // keys any slot of this workgroup can see
-  int kmin = first_visible(mask, size, ctx + t0);
-  int pos_last = ctx + (head_slots ? 1 : min(qn, t0 + 16 * tpb)) - 1;
+  // keys any slot of this workgroup can see, numbered without the gap between kept first keys and the window: number v
+  // is key v (v < kept) or key v + gap. Kept keys lie before every window here, so every valid slot sees all of them.
+  const int kfirst = first_visible(mask, size, ctx + t0);
+  const int kept = min(keep, kfirst), gap = kfirst - kept;
+  int kmin = 0;
+  int pos_last = ctx + (head_slots ? 1 : min(qn, t0 + 16 * tpb)) - 1 - gap;   // last number
   // single-token steps divide the visible key tiles over gridDim.x workgroups (merged by a second launch)
   const int nsplit = head_slots ? gridDim.x : 1;
   if (nsplit > 1) {
@@ -290,13 +304,16 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
   }
   // scores are kept in units of ln 2 (exp2 is one instruction): score * log2(e)
   constexpr float kLog2e = 1.4426950408889634f;
-  const float sc_h = scale * (temp ? temp[head] : 1.f) * kLog2e;
+  constexpr bool capped = WFN == kWeightsBounded || WFN == kWeightsCapped, bounded = WFN == kWeightsBounded;
+  // bounded scores: c tanh(z / c) = c - 2 c / (1 + e^(2 z / c)), again with 2^x: the factor below gives the exponent
+  const float cap2 = capped ? softcap * kLog2e : 0.f;
+  const float sc_h = scale * (temp ? temp[head] : 1.f) * (capped ? 2.f / softcap : 1.f) * kLog2e;
   xgk::f32x4_t o[NMT_MAX];
 #pragma unroll
   for (int mt = 0; mt < NMT_MAX; ++mt) o[mt] = xgk::f32x4_t{0.f, 0.f, 0.f, 0.f};
   // the sink starts the running softmax: weight exp(sink - m) = 1 with no value behind it
   const bool with_sink = sink && (nsplit == 1 || blockIdx.x == 0);  // the sink enters the first share only
-  float m = with_sink ? sink[head] * kLog2e : -INFINITY, l = with_sink ? 1.f : 0.f;
+  float m = bounded ? 0.f : with_sink ? sink[head] * kLog2e : -INFINITY, l = with_sink ? 1.f : 0.f;
   constexpr bool sig = WFN == kWeightsSigmoid;
   const float sbias = (sig && hbias) ? hbias[head] * kLog2e : 0.f;   // the per-head score bias, in units of ln 2
 
@@ -306,8 +323,8 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
   constexpr int NKC = (NKK_MAX * 4 + NW - 1) / NW, NVC = (NMT_MAX * 2 + NW - 1) / NW;
   uint4 sk[NKC], sv[NVC];
   auto fetch = [&](int k0) {
-    const int kabs = k0 + srow;
-    const bool ok = kabs <= pos_last;
+    const bool ok = k0 + srow <= pos_last;
+    const int kabs = k0 + srow < kept ? k0 + srow : k0 + srow + gap;
     const int64_t row = ok ? (int64_t)bt[kabs / bs] * bs + kabs % bs : 0;
     const bf16* ks = kcache + (row * G + g) * dk;
     const bf16* vs = vcache + row * G * dv_head + voff;
@@ -352,16 +369,17 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
                                       sacc[n]);
     }
     float mx = -INFINITY;
-    const bool full = slots_full && k0 + kKT - 1 <= pos_w0 && k0 >= lo_w1;
+    const bool full = slots_full && ((k0 >= kept && k0 + gap + kKT - 1 <= pos_w0 && k0 + gap >= lo_w1) || k0 + kKT <= kept);
 #pragma unroll
     for (int n = 0; n < 4; ++n)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int kabs = k0 + n * 16 + kg * 4 + r;
+        const int kv = k0 + n * 16 + kg * 4 + r, kabs = kv < kept ? kv : kv + gap;
         float v = sacc[n][r] * sc_h;
+        if constexpr (capped) v = cap2 - 2.f * cap2 * rcp_fast(1.f + exp2_fast(v));
         // r1 ln(1 + r2 d) in units of ln 2 is r1 log2(1 + r2 d)
         if (r1) v -= pen1 * __log2f(1.f + pen2 * (float)max(pos_q - kabs, 0));
-        if (!full && (!valid || kabs > pos_q || kabs < lo_q)) v = -INFINITY;
+        if (!full && (!valid || kabs > pos_q || (kabs < lo_q && kabs >= keep))) v = -INFINITY;
         sacc[n][r] = v;
         mx = fmaxf(mx, v);
       }
@@ -371,6 +389,14 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
       for (int n = 0; n < 4; ++n)
 #pragma unroll
         for (int r = 0; r < 4; ++r) sacc[n][r] = rcp_fast(1.f + exp2_fast(-(sacc[n][r] + sbias)));
+    } else if constexpr (bounded) {   // no reference needed; each lane sums its own keys, the lanes meet at the end
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          sacc[n][r] = exp2_fast(sacc[n][r]);
+          l += sacc[n][r];
+        }
     } else {
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
@@ -414,6 +440,10 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
           o[mt] = xgk::mfma16x16x32(vfrag, pfrag, o[mt]);
         }
     }
+  }
+  if constexpr (bounded) {
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
   }
   if (valid && nsplit > 1) {  // unnormalised share: (m, l) and the weighted value sum
     const int64_t row = ((int64_t)blockIdx.x * Ttot + q0 + tok) * H + head;
@@ -784,7 +814,7 @@ static int launch_masked_attention(const void* q, const void* kcache, const void
                                    const float* temp, const float* sink, void* out, int T_, int H, int G, int dk,
                                    int dv_head, int mask, int size, float scale, const void* gate, int64_t ld_gate,
                                    const float* r1, const float* r2, int vmode, int gate_elem, int wfn,
-                                   const float* hbias, hipStream_t st) {
+                                   const float* hbias, float softcap, int keep, hipStream_t st) {
   const int dv = vmode == kValuesAll ? G * dv_head : dv_head;
   int KT = 64;
   auto bytes = [&](int kt) { return ((size_t)kt * (dk + dv + 2) + (size_t)4 * kQPW * dk) * sizeof(float); };
@@ -796,7 +826,7 @@ static int launch_masked_attention(const void* q, const void* kcache, const void
                                                                block_tables, bt_width, bs, positions, token_seq, temp,
                                                                sink, (T*)out, H, G, dk, dv_head, mask, size, scale, KT,
                                                                (const T*)gate, ld_gate, r1, r2, vmode, gate_elem, wfn,
-                                                               hbias);
+                                                               hbias, softcap, keep);
   return 0;
 }
 
@@ -804,18 +834,19 @@ int masked_attention(const void* q, bool f32, const void* kcache, const void* vc
                      int bt_width, int bs, const int32_t* positions, const int32_t* token_seq, const float* temp,
                      const float* sink, void* out, int T_, int H, int G, int dk, int dv_head, int mask, int size,
                      float scale, const void* gate, int64_t ld_gate, const float* r1, const float* r2, int vmode,
-                     bool gate_elem, int wfn, const float* hbias, hipStream_t st) {
+                     bool gate_elem, int wfn, const float* hbias, float softcap, int keep, hipStream_t st) {
   if (T_ <= 0) return 0;
   const int dv = vmode == kValuesAll ? G * dv_head : dv_head;
   if (G <= 0 || H % G != 0 || dk <= 0 || dv <= 0 || dv > 512 || mask < 0 || mask > 2 ||
       (mask != kMaskCausal && size < 1) || vmode < kValuesAll || vmode >= G || (r1 && !r2) ||
-      (gate_elem && vmode != kValuesOwn) || wfn < 0 || wfn > 1 || (wfn == kWeightsSigmoid && sink))
+      (gate_elem && vmode != kValuesOwn) || wfn < 0 || wfn > 1 || (wfn == kWeightsSigmoid && (sink || softcap > 0.f)) ||
+      keep < 0 || (keep > 0 && mask != kMaskWindow))
     return -1;
 #define XGM_MA(NR)                                                                                                     \
   XGM_DISPATCH_T(f32, return (launch_masked_attention<T, NR>(q, kcache, vcache, block_tables, bt_width, bs, positions, \
                                                              token_seq, temp, sink, out, T_, H, G, dk, dv_head, mask,  \
                                                              size, scale, gate, ld_gate, r1, r2, vmode,             \
-                                                             gate_elem ? 1 : 0, wfn, hbias, st));)
+                                                             gate_elem ? 1 : 0, wfn, hbias, softcap, keep, st));)
   if (dv <= 64) { XGM_MA(1) }
   if (dv <= 128) { XGM_MA(2) }
   if (dv <= 256) { XGM_MA(4) }
@@ -829,13 +860,15 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
                           const float* sink, void* out, int T_, int ns, int max_q, int H, int G, int dk, int dv_head,
                           int mask, int size, float scale, int nsplit, float* part_o, float* part_ml, const void* gate,
                           int64_t ld_gate, const float* r1, const float* r2, int vmode, int nw_hint, bool gate_elem,
-                          int wfn, const float* hbias, hipStream_t st) {
+                          int wfn, const float* hbias, float softcap, int keep, hipStream_t st) {
   if (T_ <= 0 || ns <= 0 || max_q <= 0) return 0;
   const int dv = vmode == kValuesAll ? G * dv_head : dv_head;
   if (G <= 0 || H % G != 0 || dk % 32 != 0 || dv % 16 != 0 || dk > 128 || dv > 256 || mask < 0 || mask > 2 ||
       (mask != kMaskCausal && size < 1) || vmode < kValuesAll || vmode >= G || (r1 && !r2) ||
-      (gate_elem && vmode != kValuesOwn) || wfn < 0 || wfn > 1 || (wfn == kWeightsSigmoid && sink))
+      (gate_elem && vmode != kValuesOwn) || wfn < 0 || wfn > 1 || (wfn == kWeightsSigmoid && (sink || softcap > 0.f)) ||
+      keep < 0 || (keep > 0 && mask != kMaskWindow))
     return -1;
+  if (softcap > 0.f) wfn = (softcap * 1.4426950408889634f <= kBoundedMaxLog2 && !sink && !r1) ? kWeightsBounded : kWeightsCapped;
   const int ge = gate_elem ? 1 : 0;
   const int rep = H / G;
   const int RH = rep >= 4 ? 4 : rep >= 2 ? 2 : 1;
@@ -855,10 +888,14 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
   masked_attention_mfma_kernel<NKK, NMT, NW, WFN><<<grid, 64 * NW, lds, st>>>(                                        \
       (const bf16*)q, (const bf16*)kcache, (const bf16*)vcache, block_tables, bt_width, bs, qsl, seq_lens, slots, temp, \
       sink, (bf16*)out, H, G, dk, dv_head, mask, size, scale, RH, head_slots, part_o, part_ml, T_, (const bf16*)gate,  \
-      ld_gate, r1, r2, vmode, ge, hbias);
+      ld_gate, r1, r2, vmode, ge, hbias, softcap, keep);
 #define XGM_MK(NKK, NMT, NW)                  \
   if (wfn == kWeightsSigmoid) {               \
     XGM_MK2(NKK, NMT, NW, kWeightsSigmoid)    \
+  } else if (wfn == kWeightsBounded) {        \
+    XGM_MK2(NKK, NMT, NW, kWeightsBounded)    \
+  } else if (wfn == kWeightsCapped) {         \
+    XGM_MK2(NKK, NMT, NW, kWeightsCapped)     \
   } else {                                    \
     XGM_MK2(NKK, NMT, NW, kWeightsSoftmax)    \
   }

@@ -3,14 +3,17 @@
 //   glu_act          [gate | up] rows -> act(gate) * up':
 //                      kGluGeluTanh   0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * u
 //                      kGluClamped    g' = min(g, limit), u' = clamp(u, -limit, limit):  g' sigmoid(alpha g') (u' + 1)
-//   grouped_router   fp32 router logits -> sigmoid scores; selection score = score + correction; the experts are
-//                    split into `count` contiguous groups of equal size, a group is rated by the sum of its two
-//                    highest selection scores, members of the `keep` highest-rated groups stay eligible (all
-//                    others are excluded outright: selection score -inf); the `top` highest eligible selection
-//                    scores win; weight = score * scale (the correction does not enter it, no normalisation).
+//   grouped_router   fp32 router logits -> scores (sigmoid, or softmax over all experts); selection score = score +
+//                    correction; the experts are split into `count` contiguous groups of equal size, a group is rated
+//                    by the sum of its two highest selection scores (kRateMax: by its highest), members of the `keep`
+//                    highest-rated groups stay eligible (all others are excluded outright: selection score -inf); the
+//                    `top` highest eligible selection scores win; weight = score * scale (the correction does not
+//                    enter it, no normalisation).
 //                    For steps of few rows the logits x . rw[e] (fp32 rows and router weights) are formed here
 //                    by a four-wave workgroup per token, eight experts per sweep over the row, instead of being
 //                    read (the waves then repeat the same selection, so every barrier is met by all of them).
+//                    gate != nullptr: a logit after the experts' ones, gate[t] = sigmoid(it), takes no part in the
+//                    routing (the gate of an expert that runs for every token).
 //   moe_align        (token, choice) pairs sorted by expert into tiles of `tm` rows (padded with -1)
 //   grouped_gemm     per tile: rows x expert weights, in one of three modes:
 //                      kGemmRows    A rows as they lie in the sorted layout -> fp32 rows (the second product)
@@ -58,28 +61,46 @@ __global__ void glu_act_kernel(const T* __restrict__ in, int64_t ld, T* __restri
   }
 }
 
+// four columns per thread: rows, gate and up halves aligned to whole quads
+template <typename T>
+__global__ __launch_bounds__(256) void glu_act4_kernel(const T* __restrict__ in, int64_t ld, T* __restrict__ out, int F,
+                                                       int kind, float limit, float alpha) {
+  const int64_t t = blockIdx.y;
+  const int c = 4 * (blockIdx.x * blockDim.x + threadIdx.x);
+  if (c >= F) return;
+  float g[4], u[4];
+  ld4(in + t * ld + c, g);
+  ld4(in + t * ld + F + c, u);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) g[e] = glu(kind, g[e], u[e], limit, alpha);
+  st4(out + t * F + c, g);
+}
+
 // ------------------------------------------------------------------ router: one wave per token
 constexpr int kMaxEPL = 8;  // experts per lane: E <= 512
 
-constexpr int kRouterSweep = 8;   // experts per sweep over the row when the logits are formed here
+constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kRateTop2 = 0, kRateMax = 1;
 
+// kRouterSweep: logits per sweep over the row when they are formed here
+template <int kRouterSweep>
 __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
                                                              int E, int count, int keep, int top, float scale,
                                                              int32_t* __restrict__ ids, float* __restrict__ wts,
                                                              const float* __restrict__ x, const float* __restrict__ rw,
-                                                             int W) {
+                                                             int W, int score, int rating, float* __restrict__ gate) {
   extern __shared__ float sm[];
   float* cs = sm;              // [E] choice scores
   float* gs = sm + E;          // [count] group scores
   int* kept = (int*)(gs + count);  // [count]
-  float* lg = (float*)(kept + count);   // [E] logits formed here (x != nullptr)
-  float* part = lg + E;                 // [waves][kRouterSweep] partial sums
+  const int EL = E + (gate ? 1 : 0);    // logits per row
+  float* lg = (float*)(kept + count);   // [EL] logits formed here (x != nullptr)
+  float* part = lg + EL;                // [waves][kRouterSweep] partial sums
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const int per = E / count;
   if (x) {
     const float* xr = x + (int64_t)t * W;
     const bool vec = (W & 3) == 0;
-    for (int e0 = 0; e0 < E; e0 += kRouterSweep) {
+    for (int e0 = 0; e0 < EL; e0 += kRouterSweep) {
       float acc[kRouterSweep];
 #pragma unroll
       for (int j = 0; j < kRouterSweep; ++j) acc[j] = 0.f;
@@ -89,7 +110,7 @@ __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __rest
           ld4(xr + c, a);
 #pragma unroll
           for (int j = 0; j < kRouterSweep; ++j)
-            if (e0 + j < E) {
+            if (e0 + j < EL) {
               float b[4];
               ld4(rw + (int64_t)(e0 + j) * W + c, b);
               acc[j] += a[0] * b[0] + a[1] * b[1] + a[2] * b[2] + a[3] * b[3];
@@ -100,7 +121,7 @@ __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __rest
           const float a = xr[c];
 #pragma unroll
           for (int j = 0; j < kRouterSweep; ++j)
-            if (e0 + j < E) acc[j] += a * rw[(int64_t)(e0 + j) * W + c];
+            if (e0 + j < EL) acc[j] += a * rw[(int64_t)(e0 + j) * W + c];
         }
       }
 #pragma unroll
@@ -110,7 +131,7 @@ __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __rest
         for (int j = 0; j < kRouterSweep; ++j) part[wave * kRouterSweep + j] = acc[j];
       }
       __syncthreads();
-      if (threadIdx.x < kRouterSweep && e0 + threadIdx.x < E) {
+      if (threadIdx.x < kRouterSweep && e0 + threadIdx.x < EL) {
         float v = 0.f;
         for (int w = 0; w < nw; ++w) v += part[w * kRouterSweep + threadIdx.x];
         lg[e0 + threadIdx.x] = v;
@@ -118,26 +139,41 @@ __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __rest
       __syncthreads();
     }
   }
+  const float* lrow = x ? lg : logits + (int64_t)t * EL;
+  if (gate && threadIdx.x == 0) gate[t] = sigmoidf(lrow[E]);
   float sc[kMaxEPL], ch[kMaxEPL];
+  float mx = 0.f, inv = 1.f;
+  if (score == kScoreSoftmax) {
+    mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < kMaxEPL; ++i)
+      if (lane + 64 * i < E) mx = fmaxf(mx, lrow[lane + 64 * i]);
+    mx = wave_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxEPL; ++i)
+      if (lane + 64 * i < E) sum += expf(lrow[lane + 64 * i] - mx);
+    inv = 1.f / wave_sum(sum);
+  }
 #pragma unroll
   for (int i = 0; i < kMaxEPL; ++i) {
     const int e = lane + 64 * i;
     sc[i] = 0.f, ch[i] = -INFINITY;
     if (e < E) {
-      sc[i] = sigmoidf(x ? lg[e] : logits[(int64_t)t * E + e]);
+      sc[i] = score == kScoreSoftmax ? expf(lrow[e] - mx) * inv : sigmoidf(lrow[e]);
       ch[i] = sc[i] + (corr ? corr[e] : 0.f);
       cs[e] = ch[i];
     }
   }
   __syncthreads();
-  for (int g = lane; g < count; g += 64) {  // sum of the group's two largest choice scores
+  for (int g = lane; g < count; g += 64) {  // sum of the group's two largest choice scores, or the largest
     float a = -INFINITY, b = -INFINITY;
     for (int j = 0; j < per; ++j) {
       const float v = cs[g * per + j];
       if (v > a) b = a, a = v;
       else if (v > b) b = v;
     }
-    gs[g] = per > 1 ? a + b : a;
+    gs[g] = (per > 1 && rating == kRateTop2) ? a + b : a;
   }
   __syncthreads();
   for (int g = lane; g < count; g += 64) {  // rank among the groups (ties: the lower index first)
@@ -551,20 +587,33 @@ void glu_act(const void* in, bool f32, int64_t ld, void* out, int T_, int F, int
              hipStream_t st) {
   const int64_t total = (int64_t)T_ * F;
   if (total <= 0) return;
+  const int esz = f32 ? 4 : 2;
+  if (F % 4 == 0 && ld % 4 == 0 && (uintptr_t)in % (4 * esz) == 0 && (uintptr_t)out % (4 * esz) == 0 && T_ <= 65535) {
+    XGM_DISPATCH_T(f32, glu_act4_kernel<T><<<dim3((F / 4 + 255) / 256, T_), 256, 0, st>>>((const T*)in, ld, (T*)out, F,
+                                                                                         kind, limit, alpha);)
+    return;
+  }
   const int blocks = (int)std::min<int64_t>((total + 255) / 256, 1 << 16);
   XGM_DISPATCH_T(f32, glu_act_kernel<T><<<blocks, 256, 0, st>>>((const T*)in, ld, (T*)out, F, total, kind, limit, alpha);)
 }
 
 int grouped_router(const float* logits, const float* corr, int T_, int E, int count, int keep, int top, float scale,
-                   int32_t* ids, float* wts, const float* x, const float* rw, int W, hipStream_t st) {
+                   int32_t* ids, float* wts, const float* x, const float* rw, int W, int score, int rating, float* gate,
+                   hipStream_t st) {
   if (T_ <= 0) return 0;
   if (E < 1 || E > 64 * kMaxEPL || count < 1 || E % count != 0 || keep < 1 || keep > count || top < 1 ||
-      top > keep * (E / count))
+      top > keep * (E / count) || score < 0 || score > 1 || rating < 0 || rating > 1)
     return -1;
   if ((x != nullptr) != (rw != nullptr) || (x && W < 1) || (!x && !logits)) return -2;
   const int nth = x ? 256 : 64;
-  const size_t lds = (2 * E + 2 * count + 4 * kRouterSweep) * sizeof(float);
-  grouped_router_kernel<<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W);
+  const int EL = E + (gate ? 1 : 0);
+  const size_t lds = (E + EL + 2 * count + 4 * 16) * sizeof(float);
+  if (x && EL > 8 && EL <= 16)
+    grouped_router_kernel<16><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score,
+                                                    rating, gate);
+  else
+    grouped_router_kernel<8><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score,
+                                                   rating, gate);
   return 0;
 }
 

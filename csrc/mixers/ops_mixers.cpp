@@ -21,11 +21,12 @@ void qk_norm_cache(const void*, bool, int64_t, int, int, int, const float*, cons
                    void*, void*, int, hipStream_t);
 int masked_attention(const void*, bool, const void*, const void*, const int32_t*, int, int, const int32_t*,
                      const int32_t*, const float*, const float*, void*, int, int, int, int, int, int, int, float,
-                     const void*, int64_t, const float*, const float*, int, bool, int, const float*, hipStream_t);
+                     const void*, int64_t, const float*, const float*, int, bool, int, const float*, float, int,
+                     hipStream_t);
 int masked_attention_mfma(const void*, const void*, const void*, const int32_t*, int, int, const int32_t*, const int32_t*,
                           const int32_t*, const float*, const float*, void*, int, int, int, int, int, int, int, int, int,
                           float, int, float*, float*, const void*, int64_t, const float*, const float*, int, int, bool, int,
-                          const float*, hipStream_t);
+                          const float*, float, int, hipStream_t);
 void talk_mix(const void*, bool, const float*, const void*, int64_t, void*, int, int, int, int, hipStream_t);
 void head_norm_rope_cache(const void*, bool, int64_t, int, int, int, int, const float*, const float*, float, const float*,
                           int, int, const int32_t*, const int32_t*, void*, void*, void*, bool, int, bool, bool, const void*,
@@ -47,8 +48,12 @@ int ssm_scan(const void*, bool, int64_t, const void*, int64_t, const float*, con
 void gated_group_norm(const float*, const void*, bool, int64_t, const float*, int, float, void*, int, int, int, bool,
                       hipStream_t);
 void glu_act(const void*, bool, int64_t, void*, int, int, int, float, float, hipStream_t);
-int grouped_router(const float*, const float*, int, int, int, int, int, float, int32_t*, float*, const float*,
-                   const float*, int, hipStream_t);
+int grouped_router(const float*, const float*, int, int, int, int, int, float, int32_t*, float*, const float*, const float*,
+                   int, int, int, float*, hipStream_t);
+int hyper_residual(const float*, bool, float*, int, const void*, int64_t, bool, const float*, const float*, const int32_t*,
+                   const float*, int, const float*, const float*, const float*, const float*, float, float*, void*, bool,
+                   int, int, hipStream_t);
+void soft_cap(void*, bool, float, int64_t, hipStream_t);
 int moe_align(const int32_t*, int, int, int, int, int32_t*, int32_t*, int32_t*, hipStream_t);
 int grouped_gemm(const void*, bool, int64_t, const void*, const int32_t*, const int32_t*, int, int, int, int, int, int, void*,
                  int, float, float, const float*, bool, hipStream_t);
@@ -116,6 +121,22 @@ PYBIND11_MODULE(_mixers, m) {
                                 P<const int32_t>(dest), P<const float>(cw), top, S(st));
     check(rc, "residual_norm");
   });
+  m.def("hyper_residual", [](uintptr_t x, bool equal, uintptr_t xo, int streams, uintptr_t y1, int64_t ld1, bool y_f32,
+                             uintptr_t y_gate, uintptr_t y3, uintptr_t dest, uintptr_t cw, int top, uintptr_t w_out,
+                             uintptr_t mix, uintptr_t w_in, uintptr_t g, float eps, uintptr_t n32, uintptr_t nact,
+                             bool nact_f32, int T, int W, uintptr_t st) {
+    if (y1 && ld1 < W) throw std::invalid_argument("hyper_residual: row stride smaller than the width");
+    int rc = xgm::hyper_residual(P<const float>(x), equal, P<float>(xo), streams, P<const void>(y1), ld1, y_f32,
+                                 P<const float>(y_gate), P<const float>(y3), P<const int32_t>(dest), P<const float>(cw),
+                                 top, P<const float>(w_out), P<const float>(mix), P<const float>(w_in), P<const float>(g),
+                                 eps, P<float>(n32), P<void>(nact), nact_f32, T, W, S(st));
+    check(rc, "hyper_residual");
+  });
+  m.def("soft_cap", [](uintptr_t x, bool f32, float cap, int64_t n, uintptr_t st) {
+    if (!(cap > 0.f)) throw std::invalid_argument("soft_cap: the bound must be positive");
+    xgm::soft_cap(P<void>(x), f32, cap, n, S(st));
+    check(0, "soft_cap");
+  });
   m.def("qk_norm_cache", [](uintptr_t proj, bool f32, int64_t ld, int nq, int nk, int nv, uintptr_t wq, uintptr_t wk,
                             float eps, uintptr_t slot_mapping, uintptr_t q_out, uintptr_t kcache, uintptr_t vcache, int T,
                             uintptr_t st) {
@@ -128,14 +149,14 @@ PYBIND11_MODULE(_mixers, m) {
                                uintptr_t pos, uintptr_t token_seq, uintptr_t temp, uintptr_t sink, uintptr_t out, int T,
                                int H, int G, int dk, int dv, int mask, int size, float scale, uintptr_t gate,
                                int64_t ld_gate, uintptr_t r1, uintptr_t r2, int vmode, bool gate_elem, int wfn,
-                               uintptr_t hbias, uintptr_t st) {
+                               uintptr_t hbias, float softcap, int keep_first, uintptr_t st) {
     if (bs < 1 || bt_width < 1 || (gate && ld_gate < (gate_elem ? (int64_t)H * dv : H)))
       throw std::invalid_argument("masked_attention: inconsistent sizes");
     int rc = xgm::masked_attention(P<const void>(q), f32, P<const void>(kc), P<const void>(vc), P<const int32_t>(bt),
                                    bt_width, bs, P<const int32_t>(pos), P<const int32_t>(token_seq), P<const float>(temp),
                                    P<const float>(sink), P<void>(out), T, H, G, dk, dv, mask, size, scale,
                                    P<const void>(gate), ld_gate, P<const float>(r1), P<const float>(r2), vmode, gate_elem,
-                                   wfn, P<const float>(hbias), S(st));
+                                   wfn, P<const float>(hbias), softcap, keep_first, S(st));
     check(rc, "masked_attention");
   });
   m.def("masked_attention_mfma", [](uintptr_t q, uintptr_t kc, uintptr_t vc, uintptr_t bt, int bt_width, int bs,
@@ -143,7 +164,8 @@ PYBIND11_MODULE(_mixers, m) {
                                     uintptr_t out, int T, int ns, int max_q, int H, int G, int dk, int dv, int mask,
                                     int size, float scale, int nsplit, uintptr_t part_o, uintptr_t part_ml,
                                     uintptr_t gate, int64_t ld_gate, uintptr_t r1, uintptr_t r2, int vmode, int nw_hint,
-                                    bool gate_elem, int wfn, uintptr_t hbias, uintptr_t st) {
+                                    bool gate_elem, int wfn, uintptr_t hbias, float softcap, int keep_first,
+                                    uintptr_t st) {
     if (bs < 1 || bt_width < 1 || nsplit < 1 || (gate && ld_gate < (gate_elem ? (int64_t)H * dv : H)))
       throw std::invalid_argument("masked_attention_mfma: inconsistent sizes");
     int rc = xgm::masked_attention_mfma(P<const void>(q), P<const void>(kc), P<const void>(vc), P<const int32_t>(bt),
@@ -151,7 +173,7 @@ PYBIND11_MODULE(_mixers, m) {
                                         P<const float>(temp), P<const float>(sink), P<void>(out), T, ns, max_q, H, G, dk,
                                         dv, mask, size, scale, nsplit, P<float>(part_o), P<float>(part_ml),
                                         P<const void>(gate), ld_gate, P<const float>(r1), P<const float>(r2), vmode,
-                                        nw_hint, gate_elem, wfn, P<const float>(hbias), S(st));
+                                        nw_hint, gate_elem, wfn, P<const float>(hbias), softcap, keep_first, S(st));
     check(rc, "masked_attention_mfma");
   });
   m.def("talk_mix", [](uintptr_t o_all, bool f32, uintptr_t talk, uintptr_t gate, int64_t ld_gate, uintptr_t out, int T,
@@ -166,7 +188,8 @@ PYBIND11_MODULE(_mixers, m) {
                                    uintptr_t wk, float eps, uintptr_t rot, int rot_rows, int rot_dims, uintptr_t pos,
                                    uintptr_t slot_mapping, uintptr_t q_out, uintptr_t kc, uintptr_t vc, bool out_f32, int T,
                                    bool whole, bool half, uintptr_t v_first, int64_t ld_vf, uintptr_t v_mix, uintptr_t st) {
-    if (H < 1 || G < 1 || dk < 1 || dv < 1 || ld < (int64_t)(H + G) * dk + (int64_t)G * dv || rot_dims < 0 ||
+    if (H < 1 || G < 0 || (G > 0 && (!kc || !vc)) || dk < 1 || dv < 1 ||
+        ld < (int64_t)(H + G) * dk + (int64_t)G * dv || rot_dims < 0 ||
         rot_dims > dk || (rot_dims & 1) || (rot && rot_dims > 0 && rot_rows < 1) ||
         (v_first && (!v_mix || ld_vf < (int64_t)G * dv)))
       throw std::invalid_argument("head_norm_rope_cache: inconsistent sizes");
@@ -256,9 +279,11 @@ PYBIND11_MODULE(_mixers, m) {
     check(0, "glu_act");
   });
   m.def("grouped_router", [](uintptr_t logits, uintptr_t corr, int T, int E, int count, int keep, int top, float scale,
-                             uintptr_t ids, uintptr_t wts, uintptr_t x, uintptr_t rw, int W, uintptr_t st) {
+                             uintptr_t ids, uintptr_t wts, uintptr_t x, uintptr_t rw, int W, int score, int rating,
+                             uintptr_t gate, uintptr_t st) {
     int rc = xgm::grouped_router(P<const float>(logits), P<const float>(corr), T, E, count, keep, top, scale,
-                                 P<int32_t>(ids), P<float>(wts), P<const float>(x), P<const float>(rw), W, S(st));
+                                 P<int32_t>(ids), P<float>(wts), P<const float>(x), P<const float>(rw), W, score, rating,
+                                 P<float>(gate), S(st));
     check(rc, "grouped_router");
   });
   m.def("moe_align", [](uintptr_t ids, int pairs, int E, int cap, int tm, uintptr_t rows, uintptr_t tile_expert,

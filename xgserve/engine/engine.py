@@ -840,8 +840,8 @@ class LLMEngine:
     def export_prefix(self, tokens: Sequence[int]):
         """CacheEntry for the longest cached page-aligned prefix of `tokens` (this rank's KV shard)."""
         from .kv_io import CacheEntry
-        if self.stateful:
-            raise ValueError("prefix export needs a cache that pages alone describe")
+        if self.stateful or self.runner.kv is None:
+            raise ValueError("prefix export needs the engine's own page layout")
         with self._lock:
             blocks = self.sched.cached_prefix([int(t) for t in tokens])
             idx = torch.tensor(blocks, dtype=torch.long, device=self.device)
@@ -851,8 +851,8 @@ class LLMEngine:
 
     def import_prefix(self, entry) -> int:
         """Install a CacheEntry into the prefix cache; returns #pages newly written."""
-        if self.stateful:
-            raise ValueError("prefix import needs a cache that pages alone describe")
+        if self.stateful or self.runner.kv is None:
+            raise ValueError("prefix import needs the engine's own page layout")
         if entry.block_size != self.cfg.block_size:
             raise ValueError(f"entry block_size {entry.block_size} != engine {self.cfg.block_size}")
         want = tuple(self.runner.kv.shape[:2]) + (entry.kv.shape[2],) + tuple(self.runner.kv.shape[3:])

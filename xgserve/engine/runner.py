@@ -121,8 +121,9 @@ class ModelRunner:
         cfg = self.cfg
         self.Hkv = model.num_kv_heads_local
         # models with per-sequence state (recurrences, carried convolution inputs) or a cache
-        # layout of their own allocate it themselves: pages + one state row per sequence slot
-        self.seq_state = bool(getattr(model, "has_sequence_state", False))
+        # layout of their own allocate it themselves: pages + one state row per sequence slot.
+        # needs_seq_meta: no such state, but operators that take the step's per-sequence view
+        self.seq_state = bool(getattr(model, "has_sequence_state", False) or getattr(model, "needs_seq_meta", False))
         if hasattr(model, "alloc_cache"):
             self.kv = None
             self.kv_caches = model.alloc_cache(num_blocks, block_size, max_num_seqs)

@@ -16,7 +16,7 @@ from typing import Dict, List, Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str                      # "llama" | "mixtral" | "gpt2" | "dofivik" | "vizonex" | "loluzen" | "lotelix"
+    arch: str                      # "llama" | "mixtral" | "gpt2" | "dofivik" | "vizonex" | "loluzen" | "lotelix" | "taritar"
     hidden_size: int
     num_layers: int
     num_heads: int
@@ -46,6 +46,9 @@ class ModelConfig:
     layer_loop: Optional[dict] = None
     # "lotelix": the equal consecutive parts of a row that its RMS norms treat separately
     norm_groups: int = 1
+    # "taritar": parallel residual streams, and the bound c of logits c tanh(logits / c) (None = no bound)
+    streams: int = 1
+    logit_softcap: Optional[float] = None
 
     @property
     def q_size(self) -> int:
@@ -64,6 +67,8 @@ class ModelConfig:
                 from .loluzen import count_params
             elif self.arch == "lotelix":
                 from .lotelix import count_params
+            elif self.arch == "taritar":
+                from .taritar import count_params
             else:
                 from .dofivik import count_params
             return count_params(self)
@@ -93,9 +98,9 @@ class ModelConfig:
         if self.arch == "lotelix":
             att = [(L["mixer"].get("left") or L["mixer"]) for L in self.layer_specs if L["type"] != "mingru"]
             return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes for m in att)
-        if self.arch == "vizonex":
+        if self.arch in ("vizonex", "taritar"):   # (a layer that reads another layer's keys and values caches nothing)
             return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes
-                       for m in (L["mixer"] for L in self.layer_specs if L["type"] == "attention"))
+                       for m in (L["mixer"] for L in self.layer_specs if L["type"] == "attention") if m.get("kv_from") is None)
         if self.layer_specs is not None:
             return sum((m["kv_rank"] + m["rot_dim"]) * dtype_bytes for m in (L["mixer"] for L in self.layer_specs)
                        if "kv_rank" in m and "kv_from" not in m)
@@ -393,6 +398,95 @@ def _lotelix_tiny_layers():
 
 register(lotelix_config("lotelix-tiny", 128, 512, _lotelix_tiny_layers(), embed_scale=3.0, norm_groups=4,
                         max_position=1024))
+
+
+def taritar_config(name: str, width: int, vocab: int, layers: List[dict], streams: int = 1, embed_scale: float = 1.0,
+                   eps: float = 1e-5, logit_softcap: Optional[float] = None, max_position: int = 4096) -> ModelConfig:
+    """A Taritar model: `streams` parallel residual streams that every sublayer reads as one weighted sum and mixes when
+    it writes (hyper-connections); learned position vectors besides rotation; grouped-query attention in (2i, 2i + 1)
+    rotation pairs with bounded scores and a sliding window that also keeps the sequence's first tokens, where a layer
+    may read the cached keys and values of an earlier one; clamped-GLU feed-forwards, dense or routed (softmax scores
+    over all experts, groups rated by their best member, weights not renormalised) with a gated shared expert; bounded
+    logits."""
+    def need(d, keys, where):
+        for k in keys:
+            if k not in d:
+                raise ValueError(f"{where}: missing {k!r}")
+    if not layers:
+        raise ValueError("a model needs at least one layer")
+    if not 1 <= streams <= 32:
+        raise ValueError("streams must be in [1, 32]")
+    if width > 16384:
+        raise ValueError("widths above 16384 are not supported")
+    for i, L in enumerate(layers):
+        m, w = L.get("mixer") or {}, f"layer {i}"
+        if L.get("type") != "attention":
+            raise ValueError(f"{w}: unknown mixer type {L.get('type')!r}")
+        need(m, ("heads", "kv_heads", "dim", "vdim", "scale"), w)
+        if m["heads"] < 1 or m["kv_heads"] < 1 or m["heads"] % m["kv_heads"]:
+            raise ValueError(f"{w}: heads must be a positive multiple of kv_heads")
+        rot, mask = m.get("rot"), m.get("mask")
+        if rot is not None:
+            need(rot, ("base", "dims"), w)
+            if rot["dims"] % 2 or not 0 <= rot["dims"] <= m["dim"]:
+                raise ValueError(f"{w}: rot.dims must be even and at most dim")
+        if mask is not None:
+            need(mask, ("size",), w)
+            if mask["size"] < 1 or mask.get("keep_first", 0) < 0:
+                raise ValueError(f"{w}: mask.size must be positive and mask.keep_first not negative")
+        if m.get("softcap") is not None and m["softcap"] <= 0:
+            raise ValueError(f"{w}: softcap must be positive")
+        src = m.get("kv_from")
+        if src is not None:
+            o = layers[src]["mixer"] if 0 <= src < i else None
+            if o is None or o.get("kv_from") is not None:
+                raise ValueError(f"{w}: kv_from must name an earlier layer with keys and values of its own")
+            if any(o[k] != m[k] for k in ("kv_heads", "dim", "vdim")) or o.get("rot") != rot:
+                raise ValueError(f"{w}: kv_from layer {src} has other key / value sizes or another rotation")
+        mlp = L.get("mlp")
+        if mlp is None:
+            continue
+        if mlp.get("kind") == "dense":
+            need(mlp, ("ff", "limit"), w)
+        elif mlp.get("kind") == "moe":
+            need(mlp, ("expert", "router"), w)
+            need(mlp["expert"], ("ff", "limit"), w)
+            r = mlp["router"]
+            need(r, ("experts", "top"), w)
+            g = r.get("groups") or {"count": 1, "keep": 1}
+            E, c, k = r["experts"], g["count"], g["keep"]
+            if E < 1 or E % c or not 1 <= k <= c or not 1 <= r["top"] <= k * (E // c) or E > 512:
+                raise ValueError(f"{w}: experts must divide into groups.count groups, 1 <= keep <= count, "
+                                 "top <= keep * group size, experts <= 512")
+            if mlp.get("shared") is not None:
+                need(mlp["shared"], ("ff", "limit"), w)
+        else:
+            raise ValueError(f"{w}: unknown feed-forward kind {mlp.get('kind')!r}")
+    if logit_softcap is not None and logit_softcap <= 0:
+        raise ValueError("logit_softcap must be positive")
+    att = [L["mixer"] for L in layers]
+    ffs = [(L["mlp"]["ff"] if L["mlp"]["kind"] == "dense" else
+            L["mlp"]["expert"]["ff"] * L["mlp"]["router"]["top"] + (L["mlp"].get("shared") or {}).get("ff", 0))
+           for L in layers if L.get("mlp")]
+    return ModelConfig(name, "taritar", width, len(layers), max(m["heads"] for m in att), max(m["kv_heads"] for m in att),
+                       max(max(m["dim"], m["vdim"]) for m in att), max(ffs or [0]), vocab, max_position, 0.0, None, eps,
+                       False, bos_token_id=0, eos_token_ids=[], layer_specs=layers, embed_scale=float(embed_scale),
+                       streams=int(streams), logit_softcap=None if logit_softcap is None else float(logit_softcap))
+
+
+def _taritar_tiny_layers():
+    att = {"heads": 4, "kv_heads": 2, "dim": 32, "vdim": 16, "scale": 0.2, "softcap": 20.0,
+           "mask": {"size": 24, "keep_first": 3}, "rot": {"base": 10000.0, "dims": 16}}
+    moe = {"kind": "moe", "expert": {"ff": 32, "limit": 3.0}, "shared": {"ff": 48, "limit": 2.0},
+           "router": {"experts": 6, "top": 2, "groups": {"count": 3, "keep": 2}}}
+    return [{"type": "attention", "mixer": dict(att), "mlp": {"kind": "dense", "ff": 192, "limit": 2.5}},
+            {"type": "attention", "mixer": dict(att), "mlp": dict(moe)},
+            {"type": "attention", "mixer": dict(att, kv_from=1, mask={"size": 40}), "mlp": None},
+            {"type": "attention", "mixer": dict(att, kv_from=0), "mlp": dict(moe)}]
+
+
+register(taritar_config("taritar-tiny", 128, 512, _taritar_tiny_layers(), streams=3, embed_scale=2.0, logit_softcap=25.0,
+                        max_position=1024))
 register(ModelConfig("gpt2-tiny", "gpt2", 128, 2, 2, 2, 64, 512, 512, 256, 0.0, tie_embeddings=True,
                      bos_token_id=0, eos_token_ids=[0], dtype="float32"))
 
@@ -424,6 +518,9 @@ def from_hf_config(path: str, name: Optional[str] = None) -> ModelConfig:
     if c.get("architecture") == "Lotelix":
         return lotelix_config(name or "lotelix", c["width"], c["vocab"], c["layers"], c["embedding"]["scale"],
                               c["norm"]["eps"], int(c["norm"].get("groups", 1)), int(c.get("max_position", 131072)))
+    if c.get("architecture") == "Taritar":
+        return taritar_config(name or "taritar", c["width"], c["vocab"], c["layers"], int(c["streams"]),
+                              c["embedding"]["scale"], c["norm"]["eps"], c.get("logit_softcap"), int(c["max_positions"]))
     mt = c.get("model_type", "llama")
     eos = c.get("eos_token_id", 2)
     eos = eos if isinstance(eos, list) else [eos]

@@ -24,12 +24,13 @@ from .gpt2 import GPT2ForCausalLM
 from .llama import LlamaForCausalLM
 from .loluzen import LoluzenForCausalLM
 from .lotelix import LotelixForCausalLM
+from .taritar import TaritarForCausalLM
 from .vizonex import VizonexForCausalLM
 
 
 def model_class(cfg: ModelConfig):
     return {"gpt2": GPT2ForCausalLM, "dofivik": DofivikForCausalLM, "vizonex": VizonexForCausalLM,
-            "loluzen": LoluzenForCausalLM, "lotelix": LotelixForCausalLM}.get(cfg.arch, LlamaForCausalLM)
+            "loluzen": LoluzenForCausalLM, "lotelix": LotelixForCausalLM, "taritar": TaritarForCausalLM}.get(cfg.arch, LlamaForCausalLM)
 
 
 def _resolve_shapes(cfg: ModelConfig, checkpoint: str) -> None:
@@ -143,6 +144,8 @@ def load_checkpoint(model, path: str) -> None:
         _load_loluzen(model, r)
     elif cfg.arch == "lotelix":
         _load_lotelix(model, r)
+    elif cfg.arch == "taritar":
+        _load_taritar(model, r)
     else:
         _load_llama(model, r)
 
@@ -434,6 +437,70 @@ def _save_lotelix(model, path: str) -> None:
                    "norm": {"eps": cfg.norm_eps, "groups": cfg.norm_groups}, "max_position": cfg.max_position}, f, indent=1)
 
 
+def _taritar_tensors(m):
+    """(checkpoint name, parameter, index of a fused / stacked parameter or None) for every tensor."""
+    out = [("embed", m.embed, None), ("pos", m.pos, None), ("head", m.head, None), ("final.norm", m.final_norm, None)]
+
+    def glu(pre, mod):
+        F_ = mod.ff
+        return [(pre + "gate", mod.gate_up, slice(0, F_)), (pre + "up", mod.gate_up, slice(F_, 2 * F_)),
+                (pre + "down", mod.down, None)]
+
+    def hyper(pre, hc):
+        return [(pre + "in", hc.w_in, None), (pre + "out", hc.w_out, None), (pre + "mix", hc.mix, None)]
+    for i, L in enumerate(m.layers):
+        b, x = f"l{i}.", L.mix
+        out.append((b + "norm1", L.norm1, None))
+        out += hyper(b + "hc1.", L.hc1)
+        out.append((b + "mix.q", x.in_proj, slice(0, x.nq)))
+        if x.kv_from is None:
+            out += [(b + "mix.k", x.in_proj, slice(x.nq, x.nq + x.nk)), (b + "mix.v", x.in_proj, slice(x.nq + x.nk, None))]
+        out.append((b + "mix.o", x.o, None))
+        if L.mlp is None:
+            continue
+        out.append((b + "norm2", L.norm2, None))
+        out += hyper(b + "hc2.", L.hc2)
+        if not L.moe:
+            out += glu(b + "mlp.", L.mlp)
+            continue
+        F_, E = L.mlp.ff, L.mlp.E
+        out.append((b + "mlp.router", L.mlp.router, slice(0, E)))
+        for e in range(E):
+            out += [(f"{b}mlp.e{e}.gate", L.mlp.w13, (e, slice(0, F_))), (f"{b}mlp.e{e}.up", L.mlp.w13, (e, slice(F_, 2 * F_))),
+                    (f"{b}mlp.e{e}.down", L.mlp.w2, e)]
+        if L.mlp.shared is not None:
+            out += glu(b + "mlp.shared.", L.mlp.shared)
+            out.append((b + "mlp.shared.sg", L.mlp.router, slice(E, E + 1)))
+    return out
+
+
+def _load_taritar(m, r: _Reader):
+    """Tensors `embed`, `pos`, `head`, `final.norm`, `l<i>.<norm1|norm2>`, `l<i>.<hc1|hc2>.<in|out|mix>`, `l<i>.mix.*`,
+    `l<i>.mlp.*` ([out, in] matrices). q / k / v and gate / up are fused row-wise, the experts stacked, the shared
+    expert's gate appended to the router's rows, on load."""
+    for name, p, idx in _taritar_tensors(m):
+        src = r.get(name)
+        dst = p.data if idx is None else p.data[idx]
+        if tuple(dst.shape) != tuple(src.shape):
+            raise ValueError(f"shape mismatch for {name}: model {tuple(dst.shape)} vs checkpoint {tuple(src.shape)}")
+        dst.copy_(src.to(dst.dtype))
+
+
+def _save_taritar(model, path: str) -> None:
+    from safetensors.torch import save_file
+    cfg = model.cfg
+    t = {}
+    for name, p, idx in _taritar_tensors(model):
+        v = p.data if idx is None else p.data[idx]
+        t[name] = v.detach().to(torch.bfloat16).contiguous().cpu()
+    save_file(t, os.path.join(path, "model.safetensors"))
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump({"architecture": "Taritar", "width": cfg.hidden_size, "vocab": cfg.vocab_size,
+                   "embedding": {"scale": cfg.embed_scale}, "streams": cfg.streams, "layers": cfg.layer_specs,
+                   "norm": {"eps": cfg.norm_eps}, "logit_softcap": cfg.logit_softcap,
+                   "max_positions": cfg.max_position}, f, indent=1)
+
+
 def _save_vizonex(model, path: str) -> None:
     from safetensors.torch import save_file
     cfg = model.cfg
@@ -481,6 +548,8 @@ def save_checkpoint(model, path: str) -> None:
         return _save_loluzen(model, path)
     if cfg.arch == "lotelix":
         return _save_lotelix(model, path)
+    if cfg.arch == "taritar":
+        return _save_taritar(model, path)
     t: Dict[str, torch.Tensor] = {}
     if cfg.arch == "gpt2":
         t["transformer.wte.weight"] = model.wte

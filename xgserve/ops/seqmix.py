@@ -460,6 +460,78 @@ def residual_norm(x: torch.Tensor, y1: Optional[torch.Tensor], a1: Optional[torc
     return n32, nact
 
 
+# ---------------------------------------------------------------------------- several residual streams
+def hyper_residual(x: torch.Tensor, streams: int, y1: Optional[torch.Tensor], y3, w_out: Optional[torch.Tensor],
+                   mix: Optional[torch.Tensor], w_in: Optional[torch.Tensor], norm_w: torch.Tensor, eps: float,
+                   out_dtype: torch.dtype, want_f32: bool = False, y_gate: Optional[torch.Tensor] = None,
+                   store: bool = True):
+    """One sublayer's write to the residual streams and the next one's read, per token:
+        y   = y1 * y_gate + y3                                  (either may be None; y_gate None = 1)
+        x_t <- sum_s mix[s, t] x_s + w_out[t] y                 (all from the old streams; skipped when mix is None)
+        n   = N(sum_s w_in[s] x_s) * norm_w                     (w_in None = ones; N(v) = v / sqrt(mean(v^2) + eps))
+    x fp32 [T, S, W], or [T, W] when all S = `streams` streams are equal (a sequence's start); y1 [T, W] activation
+    tensor; y_gate fp32 [T]; y3 fp32 [T, W] or the `RoutedRows` of routed_experts(combine=False); w_out / w_in fp32 [S];
+    mix fp32 [S, S] ([from, to]). Returns (x [T, S, W], n fp32 or None, n as out_dtype); x is updated in place where it
+    has its streams; with store=False the new streams are not kept (x is returned as it came)."""
+    T, W, S = x.shape[0], x.shape[-1], int(streams)
+    assert x.dim() == 2 or x.shape[1] == S
+    routed = None
+    if isinstance(y3, RoutedRows):
+        if y3.dest is None:
+            y3 = y3.y
+        else:
+            routed, y3 = y3, y3.y
+    if not native_device(x):
+        X = x if x.dim() == 3 else x[:, None, :].expand(T, S, W)
+        if mix is not None:
+            if routed is not None:
+                rows = y3[routed.dest.long()]
+                y3 = (rows * routed.wts[:, :, None]).sum(1) if routed.wts is not None else rows.sum(1)
+            y = torch.zeros(T, W)
+            if y1 is not None:
+                y = y + (y1.float() if y_gate is None else y1.float() * y_gate[:, None])
+            if y3 is not None:
+                y = y + y3
+            X = torch.einsum("tsw,sr->trw", X, mix) + w_out[None, :, None] * y[:, None, :]
+            if store:
+                x = x.copy_(X) if x.dim() == 3 else X
+        u = X.sum(1) if w_in is None else (X * w_in[None, :, None]).sum(1)
+        n = u / torch.sqrt(u.pow(2).mean(-1, keepdim=True) + eps) * norm_w
+        return x, (n if want_f32 else None), n.to(out_dtype)
+    assert x.dtype == torch.float32 and x.is_contiguous() and norm_w.numel() == W
+    assert (mix is None) == (w_out is None) and (mix is not None or (y1 is None and y3 is None))
+    for t, n_ in ((mix, S * S), (w_out, S), (w_in, S), (norm_w, W)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n_)
+    assert y1 is None or (y1.stride(1) == 1 and y1.shape == (T, W))
+    assert y_gate is None or (y1 is not None and y_gate.dtype == torch.float32 and y_gate.is_contiguous() and y_gate.numel() == T)
+    assert y3 is None or (y3.dtype == torch.float32 and y3.is_contiguous() and y3.shape[1] == W)
+    if routed is not None:
+        assert routed.dest.dtype == torch.int32 and routed.dest.is_contiguous() and routed.dest.shape[0] == T
+        assert routed.wts is None or (routed.wts.is_contiguous() and routed.wts.shape == routed.dest.shape)
+    else:
+        assert y3 is None or y3.shape[0] == T
+    out = x
+    if mix is not None and store and x.dim() == 2:
+        out = torch.empty(T, S, W, dtype=torch.float32, device=x.device)
+    n32 = torch.empty(T, W, dtype=torch.float32, device=x.device) if want_f32 else None
+    nact = torch.empty(T, W, dtype=out_dtype, device=x.device)
+    mixers().hyper_residual(x.data_ptr(), x.dim() == 2, _p(out) if (mix is not None and store) else 0, S, _p(y1),
+                            y1.stride(0) if y1 is not None else 0, is_f32(y1) if y1 is not None else True, _p(y_gate),
+                            _p(y3), _p(routed.dest) if routed else 0, _p(routed.wts) if routed else 0,
+                            routed.dest.shape[1] if routed else 0, _p(w_out), _p(mix), _p(w_in), norm_w.data_ptr(),
+                            float(eps), _p(n32), nact.data_ptr(), is_f32(nact), T, W, stream_ptr())
+    return out, n32, nact
+
+
+def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """x <- cap * tanh(x / cap), in place (formed in fp32)."""
+    if not native_device(x):
+        return x.copy_(cap * torch.tanh(x.float() / cap))
+    assert x.is_contiguous()
+    mixers().soft_cap(x.data_ptr(), is_f32(x), float(cap), x.numel(), stream_ptr())
+    return x
+
+
 # ---------------------------------------------------------------------------- grouped-query attention, masked
 MASK_CAUSAL, MASK_WINDOW, MASK_CHUNK = 0, 1, 2
 # XGS_TUNE attn_mfma=0: the general (any size, fp32-capable) kernel for bf16 too (A/B and tests)
@@ -515,10 +587,12 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                      mask: int, size: int, scale: float, temp: Optional[torch.Tensor], sink: Optional[torch.Tensor],
                      block_size: int, sm: SeqMeta, gate: Optional[torch.Tensor] = None,
                      dist: Optional[tuple] = None, values: int = V_OWN, gate_elem: bool = False,
-                     weights: int = W_SOFTMAX, score_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     weights: int = W_SOFTMAX, score_bias: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                     keep_first: int = 0) -> torch.Tensor:
     """Softmax attention of H query heads over G cached key/value heads (query head h reads head h // (H / G)).
-    A query at position i sees keys first_visible(mask, size, i) .. i of its own sequence. score = (q . k) * scale
-    * temp[h]; with `dist` = (r1, r2) (fp32 [H] each) the score of key j loses r1[h] * ln(1 + r2[h] * (i - j)),
+    A query at position i sees keys first_visible(mask, size, i) .. i of its own sequence, and with `keep_first` (sliding
+    windows) also the sequence's first keep_first keys up to its own position. score = (q . k) * scale * temp[h], with
+    `softcap` > 0 bounded to softcap * tanh(score / softcap); with `dist` = (r1, r2) (fp32 [H] each) the score of key j loses r1[h] * ln(1 + r2[h] * (i - j)),
     otherwise positions do not enter the scores; with `sink` the denominator also holds exp(sink[h]), a term with no
     key and no value; with `gate` ([T, >= H], row-strided) head h's output is multiplied by sigmoid(gate[t, h]), or,
     with `gate_elem` (gate [T, >= H dv]), entry d of head h by sigmoid(gate[t, h dv + d]).
@@ -538,6 +612,8 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                                 gate.shape[1] >= (H * dv if gate_elem else H))
         assert not gate_elem or values == V_OWN
         assert weights == W_SOFTMAX or (sink is None and weights == W_SIGMOID)
+        assert keep_first == 0 or mask == MASK_WINDOW
+        assert softcap == 0 or weights == W_SOFTMAX
         assert score_bias is None or (score_bias.dtype == torch.float32 and score_bias.numel() == H)
         r1, r2 = dist if dist is not None else (None, None)
         bt = _i32(sm.block_tables)
@@ -548,7 +624,7 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
             # single tokens as the query heads of one key/value head per wave
             nsplit, part_o, part_ml = 1, None, None
             if single:  # divide the visible key tiles over several workgroups (merged by a second launch)
-                tiles = (size + 63) // 64 if mask != MASK_CAUSAL else ATTN_MAX_SPLITS
+                tiles = (size + keep_first + 63) // 64 if mask != MASK_CAUSAL else ATTN_MAX_SPLITS
                 nsplit = max(1, min(ATTN_MAX_SPLITS, tiles, ATTN_SPLIT_WGS // max(1, T * G)))
                 if nsplit > 1:
                     part_o = torch.empty(nsplit * T * H * dvo, dtype=torch.float32, device=q.device)
@@ -559,13 +635,14 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                                            sm.max_q, H, G, dk, dv, int(mask), int(size), float(scale), nsplit,
                                            _p(part_o), _p(part_ml), _p(gate), gate.stride(0) if gate is not None else 0,
                                            _p(r1), _p(r2), int(values), ATTN_WAVES, bool(gate_elem), int(weights),
-                                           _p(score_bias), stream_ptr())
+                                           _p(score_bias), float(softcap), int(keep_first), stream_ptr())
             return out
         mixers().masked_attention(q.data_ptr(), is_f32(q), kcache.data_ptr(), vcache.data_ptr(), bt.data_ptr(),
                                   bt.shape[1], block_size, _i32(sm.positions).data_ptr(), _i32(sm.token_seq).data_ptr(),
                                   _p(temp), _p(sink), out.data_ptr(), T, H, G, dk, dv, int(mask), int(size), float(scale),
                                   _p(gate), gate.stride(0) if gate is not None else 0, _p(r1), _p(r2), int(values),
-                                  bool(gate_elem), int(weights), _p(score_bias), stream_ptr())
+                                  bool(gate_elem), int(weights), _p(score_bias), float(softcap), int(keep_first),
+                                  stream_ptr())
         return out
     kr, vr = kcache.view(-1, G, dk), vcache.view(-1, G, dv)
     qf = q.float().view(T, H, dk)
@@ -577,10 +654,13 @@ def masked_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
         if s < 0:
             out[t] = 0
             continue
-        keys = torch.arange(first_visible(mask, size, pos[t]), pos[t] + 1)
+        lo = first_visible(mask, size, pos[t])
+        keys = torch.cat([torch.arange(min(keep_first, lo)), torch.arange(lo, pos[t] + 1)])
         idx = sm.block_tables[s][(keys // block_size).long()].long() * block_size + keys % block_size
         kk = kr[idx].float().repeat_interleave(rep, 1)   # [n, H, dk]
         sc = torch.einsum("hd,nhd->hn", qf[t], kk) * (scale * tmp)[:, None]
+        if softcap:
+            sc = softcap * torch.tanh(sc / softcap)
         if dist is not None:
             sc = sc - dist[0][:, None] * torch.log1p(dist[1][:, None] * (pos[t] - keys).float()[None, :])
         if weights == W_SIGMOID:
@@ -705,15 +785,22 @@ ROUTER_FUSED_MAX_WORK = 16384   # ... when experts x width stays within this (me
                                 # 8 x 2048, 20 against 16 us at 8 x 4096)
 
 
+SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1   # grouped_router(score=...)
+RATE_TOP2, RATE_MAX = 0, 1            # grouped_router(rating=...): how a group of experts is rated
+
+
 def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Tensor], count: int, keep: int, top: int,
-                   scale: float, rows: Optional[torch.Tensor] = None, router_w: Optional[torch.Tensor] = None):
+                   scale: float, rows: Optional[torch.Tensor] = None, router_w: Optional[torch.Tensor] = None,
+                   score: int = SCORE_SIGMOID, rating: int = RATE_TOP2, extra_gate: bool = False, want_gate: bool = False):
     """fp32 router logits [T, E] -> (expert ids int32 [T, top], weights fp32 [T, top]). With `rows` (fp32 [T, W]) and
     `router_w` (fp32 [E, W]) in place of `logits` the logits are rows . router_w[e] in fp32: inside the router kernel
     for steps of few rows on the GPU (a launch less; the library product wins on long steps), else a matrix product. Scores are
-    sigmoid(logits). Selection uses score + correction: the experts form `count` contiguous groups of equal
-    size, a group is rated by the sum of its two highest selection scores, and only members of the `keep`
-    highest-rated groups are eligible (everything else is excluded outright, selection score -inf). The
-    returned weights are score * scale: the correction does not enter them and they are not normalised."""
+    sigmoid(logits), or with SCORE_SOFTMAX their softmax over all experts. Selection uses score + correction: the experts form `count` contiguous groups of equal
+    size, a group is rated by the sum of its two highest selection scores (RATE_MAX: by its highest), and only members of
+    the `keep` highest-rated groups are eligible (everything else is excluded outright, selection score -inf). The
+    returned weights are score * scale: the correction does not enter them and they are not normalised.
+    `extra_gate`: the logits (or router_w) hold one entry more than there are experts, the logit of a gate that is
+    independent of the routing; with `want_gate` (ids, weights, sigmoid(gate) fp32 [T] or None) is returned."""
     fused = False
     if logits is None:
         assert rows.dtype == router_w.dtype == torch.float32 and rows.shape[1] == router_w.shape[1]
@@ -722,24 +809,30 @@ def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Te
         if not fused:
             logits = torch.nn.functional.linear(rows, router_w)
     T, E = (rows.shape[0], router_w.shape[0]) if fused else logits.shape
+    E -= int(extra_gate)
     if not fused and not native_device(logits):
-        s = torch.sigmoid(logits.float())
+        gate = torch.sigmoid(logits[:, E].float()) if extra_gate else None
+        z = logits[:, :E].float()
+        s = torch.softmax(z, -1) if score == SCORE_SOFTMAX else torch.sigmoid(z)
         c = s + (correction if correction is not None else 0.0)
         per = E // count
-        gsc = c.view(T, count, per).topk(min(2, per), -1).values.sum(-1)
+        gsc = c.view(T, count, per).topk(1 if rating == RATE_MAX else min(2, per), -1).values.sum(-1)
         kept = torch.zeros(T, count, dtype=torch.bool)
         kept.scatter_(1, gsc.topk(keep, -1).indices, True)
         c = c.masked_fill(~kept.repeat_interleave(per, 1), float("-inf"))
         ids = c.topk(top, -1).indices
-        return ids.to(torch.int32), s.gather(1, ids) * scale
+        ids, wts = ids.to(torch.int32), s.gather(1, ids) * scale
+        return (ids, wts, gate) if want_gate else (ids, wts)
     assert fused or (logits.dtype == torch.float32 and logits.is_contiguous())
     dev = rows.device if fused else logits.device
     ids = torch.empty(T, top, dtype=torch.int32, device=dev)
     wts = torch.empty(T, top, dtype=torch.float32, device=dev)
+    gate = torch.empty(T, dtype=torch.float32, device=dev) if extra_gate else None
     mixers().grouped_router(0 if fused else logits.data_ptr(), _p(correction), T, E, int(count), int(keep), int(top),
                             float(scale), ids.data_ptr(), wts.data_ptr(), rows.data_ptr() if fused else 0,
-                            router_w.data_ptr() if fused else 0, rows.shape[1] if fused else 0, stream_ptr())
-    return ids, wts
+                            router_w.data_ptr() if fused else 0, rows.shape[1] if fused else 0, int(score), int(rating),
+                            _p(gate), stream_ptr())
+    return (ids, wts, gate) if want_gate else (ids, wts)
 
 
 def _act_ref(z, kind):
@@ -869,14 +962,17 @@ def head_norm_rope_cache(src: torch.Tensor, H: int, G: int, dk: int, dv: int, wq
     entry i with i + rot_dims / 2) by the table row of the token's position (rot fp32 [positions, rot_dims / 2, 2],
     None = no rotation). With `v_first` ([T, G dv], row-strided, the values another layer projected for the same
     tokens) and `v_mix` (fp32, one element, lambda) the values become (1 - lambda) v + lambda v_first. q is returned
-    [T, H dk]; k and the (mixed) v go to cache rows slot_mapping[t]."""
+    [T, H dk]; k and the (mixed) v go to cache rows slot_mapping[t]. G = 0: rows of queries alone, nothing is cached
+    (kcache / vcache None)."""
     T = src.shape[0]
     nq, nk, nv = H * dk, G * dk, G * dv
     q = torch.empty(T, nq, dtype=out_dtype, device=src.device)
     assert (v_first is None) == (v_mix is None)
     if native_device(src):
-        assert src.stride(1) == 1 and kcache.is_contiguous() and vcache.is_contiguous()
-        assert kcache.dtype == vcache.dtype == out_dtype and kcache.shape[-1] == nk and vcache.shape[-1] == nv
+        assert src.stride(1) == 1
+        if G:
+            assert kcache.is_contiguous() and vcache.is_contiguous()
+            assert kcache.dtype == vcache.dtype == out_dtype and kcache.shape[-1] == nk and vcache.shape[-1] == nv
         assert rot is None or (rot.dtype == torch.float32 and rot.is_contiguous() and rot.shape[1] * 2 == rot_dims)
         assert rot_dims % 2 == 0 and rot_dims <= dk
         assert not whole or ((wq is None or wq.numel() == nq) and (wk is None or wk.numel() == nk))
@@ -886,8 +982,8 @@ def head_norm_rope_cache(src: torch.Tensor, H: int, G: int, dk: int, dv: int, wq
         mixers().head_norm_rope_cache(src.data_ptr(), is_f32(src), src.stride(0), H, G, dk, dv, _p(wq), _p(wk),
                                       float(eps), _p(rot), rot.shape[0] if rot is not None else 0,
                                       rot_dims if rot is not None else 0, _i32(sm.positions).data_ptr(),
-                                      _i32(sm.slot_mapping).data_ptr(), q.data_ptr(), kcache.data_ptr(),
-                                      vcache.data_ptr(), is_f32(q), T, bool(whole), bool(half), _p(v_first),
+                                      _i32(sm.slot_mapping).data_ptr(), q.data_ptr(), _p(kcache) if G else 0,
+                                      _p(vcache) if G else 0, is_f32(q), T, bool(whole), bool(half), _p(v_first),
                                       v_first.stride(0) if v_first is not None else 0, _p(v_mix), stream_ptr())
         return q
     pf = src.float()
@@ -902,6 +998,8 @@ def head_norm_rope_cache(src: torch.Tensor, H: int, G: int, dk: int, dv: int, wq
             v = _rotate_pairs(v, rot, sm.positions, rot_dims, half)
         return v.reshape(T, n * dk)
     q.copy_(prep(pf[:, :nq], H, wq).to(out_dtype))
+    if G == 0:
+        return q
     ok = sm.slot_mapping >= 0
     rows = sm.slot_mapping[ok].long()
     kcache.view(-1, nk)[rows] = prep(pf[:, nq:nq + nk], G, wk)[ok].to(kcache.dtype)
