@@ -84,6 +84,9 @@ class SpeculativeDecoder:
             self.model, dcfg = draft_model, draft_model.cfg
         if dcfg.vocab_size != engine.mcfg.vocab_size:
             raise ValueError(f"draft vocab {dcfg.vocab_size} != target vocab {engine.mcfg.vocab_size}")
+        if getattr(self.model, "has_sequence_state", False):
+            raise ValueError(f"draft model {dcfg.name}: a per-sequence recurrent state cannot be rolled back to the "
+                             "accepted tokens")
         ec = engine.cfg
         bs = ec.block_size
         per_seq = (engine.max_model_len + bs - 1) // bs + 1
@@ -173,7 +176,8 @@ class SpeculativeDecoder:
                 "max_q_len": max(ql), "bt_width": w, "input_ids": i32(ids), "positions": i32(pos),
                 "slot_mapping": i32(slot), "q_lens": i32(ql), "seq_lens": i32(sl), "query_start_loc": i32(qsl),
                 "block_tables": bt.reshape(-1), "logits_indices": i32(li), "is_embed": np.zeros(ns, np.uint8),
-                "order": rows}
+                # drafts keep everything in their pages: the slots only say that no row is padding
+                "slots": np.arange(ns, dtype=np.int32), "order": rows}
 
     def propose(self) -> None:
         """Called by the engine (under its lock) right before scheduling."""
