@@ -162,8 +162,8 @@ def random_weights(cfg, seed=0):
         out[name] = torch.randn(n, generator=g) * std + mean
 
     def glu(pre, ff):
-        mat(pre + "gate", ff, W, 1.5)
-        mat(pre + "up", ff, W, 1.5)
+        mat(pre + "gate", ff, W)
+        mat(pre + "up", ff, W)
         mat(pre + "down", W, ff)
 
     def hyper(pre):
@@ -179,9 +179,9 @@ def random_weights(cfg, seed=0):
         H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
         vec(pre + "norm1", W, 0.2, 1.0)
         hyper(pre + "hc1.")
-        mat(pre + "mix.q", H * dk, W, 2.0)
+        mat(pre + "mix.q", H * dk, W, 1.2)
         if m.get("kv_from") is None:
-            mat(pre + "mix.k", G * dk, W, 2.0)
+            mat(pre + "mix.k", G * dk, W, 1.2)
             mat(pre + "mix.v", G * dv, W)
         mat(pre + "mix.o", W, H * dv)
         if mlp is None:
@@ -191,7 +191,7 @@ def random_weights(cfg, seed=0):
         if mlp["kind"] == "dense":
             glu(pre + "mlp.", mlp["ff"])
             continue
-        mat(pre + "mlp.router", mlp["router"]["experts"], W, 3.0)
+        mat(pre + "mlp.router", mlp["router"]["experts"], W, 2.0)
         for e in range(mlp["router"]["experts"]):
             glu(f"{pre}mlp.e{e}.", mlp["expert"]["ff"])
         if mlp.get("shared"):
