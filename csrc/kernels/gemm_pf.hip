@@ -40,19 +40,23 @@
 //     partials [S, M, N] reduced by the consumer (rope_cache_partials /
 //     add_partials_rmsnorm), like every other projection kernel here.
 // Epilogues: bf16, fp32 partials, or silu(gate) * up of a block-16 interleaved
-// gate|up weight (the SiLU-gate fused: no [M, 2F] intermediate).
+// gate|up weight (the SiLU-gate fused: no [M, 2F] intermediate). PF_GLU (grouped form
+// only): a gated activation of glu.h on a weight whose gate rows come first and whose up
+// rows follow ([gate F | up F]): the W tile's DMA takes 16 gate rows and the 16 up rows of
+// the same columns alternately, so the LDS image and the epilogue are the interleaved ones.
 // Grouped form (gemm_pf_grouped, GRP): the prompt-sized expert GEMMs of an MoE layer
 // over moe_align's expert-sorted rows -- one tile per expert segment, so each expert's
 // weights stream once per step (profiles/r5_moe_pf.md).
 #include <type_traits>
 
 #include "glds.h"
+#include "glu.h"
 
 namespace xgk {
 
 int k_rotation(int S);  // gemm_m64g.hip
 
-enum : int { PF_BF16 = 0, PF_PARTIAL = 1, PF_SILU = 2 };
+enum : int { PF_BF16 = 0, PF_PARTIAL = 1, PF_SILU = 2, PF_GLU = 3 };
 constexpr int PF_GROUP_M = 8;  // M tiles per group of the tile order
 // K-tile rotation per W tile (set_pf_krot(1); off by default): it spreads the
 // lock-step HBM stream of the weight-streaming kernels, but here it would put the
@@ -142,7 +146,7 @@ __device__ __forceinline__ void pf_wait(bool steady) {
 // 64-padded row space [P]; expert e owns rows [offs[e], offs[e + 1]) and its own
 // weight w + e * w_stride. Tile slot mi of a column tile walks the experts' tiles in
 // order (expert e has ceil(segment / BM) of them); slots past the last tile exit.
-// A row p of a tile reads x row rows[p] (rows == nullptr: row p; -1 = a pad: row 0,
+// A row p of a tile reads x row rows[p] / top (rows == nullptr: row p; -1 = a pad: row 0,
 // finite data never combined), rows past the segment end are not stored.
 struct PfGrp {
   const int32_t* rows;
@@ -150,9 +154,13 @@ struct PfGrp {
   int E;
   int mt;            // tile slots per column tile (host bound on the experts' tiles)
   int64_t w_stride;  // elements between two experts' [N, K] weights
+  int top;           // rows[] holds token * top + choice (1: the token itself)
+  int kind;          // PF_GLU: the gated activation and its constants
+  float limit, alpha;
 };
 
-template <int BM, int MTP, bool NT, int PR = 0, int LAG = 1, bool GRP = false>
+// SPLIT (GRP): PF_GLU's [gate F | up F] weight
+template <int BM, int MTP, bool NT, int PR = 0, int LAG = 1, bool GRP = false, bool SPLIT = false>
 __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restrict__ x, int M, int K,
                                                           const uint16_t* __restrict__ w, int N, int S,
                                                           float* __restrict__ part, uint16_t* __restrict__ out,
@@ -228,12 +236,13 @@ __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restr
       for (int q = 0; q < P; ++q) {
         int row = min(m0 + r + 16 * MTP * q, m_hi - 1);
         if constexpr (GRP) {
-          if (grp.rows != nullptr) row = max(grp.rows[row], 0);
+          if (grp.rows != nullptr) row = max(grp.rows[row], 0) / grp.top;
         }
         asrc[q][a] = x + static_cast<int64_t>(row) * K + sw;
       }
     }
-    const uint16_t* bsrc = wb + static_cast<int64_t>(n0 + 32 * wid + dr) * K + sw;  // + 8 i rows per piece
+    // + 8 i rows per piece; SPLIT: pieces 0 / 1 are 16 gate rows, 2 / 3 the same 16 up rows, N / 2 rows further on
+    const uint16_t* bsrc = wb + static_cast<int64_t>(SPLIT ? n0 / 2 + 16 * wid + dr : n0 + 32 * wid + dr) * K + sw;
     auto kof = [&](int t) {
       const int tt = t + rot;
       return (kt_lo + (tt >= nk ? tt - nk : tt)) * 64;
@@ -247,7 +256,7 @@ __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restr
     };
     auto issue_b = [&](int t, int i) {
       if constexpr (PR == 1) return;
-      const uint16_t* src = bsrc + static_cast<int64_t>(8 * i) * K + kof(t);
+      const uint16_t* src = bsrc + static_cast<int64_t>(SPLIT ? 8 * (i & 1) + (i >> 1) * (N / 2) : 8 * i) * K + kof(t);
       uint8_t* dst = smem + (t & 1) * SLOT + ASZ + (4 * wid + i) * 1024;
       if constexpr (NT) glds16_nt(src, dst);
       else glds16(src, dst);
@@ -380,7 +389,7 @@ __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restr
           }
         }
     } else {
-      // SiLU gate: n tiles 2j (gate) / 2j + 1 (up) are one interleaved 16-row block pair
+      // SiLU gate (SPLIT: the gated activation of grp.kind): n tiles 2j (gate) / 2j + 1 (up) are one interleaved 16-row block pair
       const int F = N / 2, f0 = (n0 + wrow) / 2 + 4 * g;
 #pragma unroll
       for (int q = 0; q < P; ++q)
@@ -394,7 +403,8 @@ __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restr
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const float gt = acc[q][mt][2 * j][r];
-              o[r] = gt / (1.f + __expf(-gt)) * acc[q][mt][2 * j + 1][r];
+              if constexpr (SPLIT) o[r] = glu(grp.kind, gt, acc[q][mt][2 * j + 1][r], grp.limit, grp.alpha);
+              else o[r] = gt / (1.f + __expf(-gt)) * acc[q][mt][2 * j + 1][r];
             }
             uint2 v2;
             v2.x = pack2(o[0], o[1]);
@@ -442,7 +452,7 @@ __global__ void __launch_bounds__(512, 1) gemm_pf_kernel(const uint16_t* __restr
 template <int BM, int MTP, bool NT, int PR = 0, int LAG = 1>
 static int launch_pf(int tiles, hipStream_t st, const uint16_t* x, int M, int K, const uint16_t* w, int N, int S,
                      float* part, uint16_t* out, int mode) {
-  const PfGrp ng{nullptr, nullptr, 0, 0, 0};
+  const PfGrp ng{nullptr, nullptr, 0, 0, 0, 1, 0, 0.f, 0.f};
   hipLaunchKernelGGL((gemm_pf_kernel<BM, MTP, NT, PR, LAG>), dim3(tiles * S), dim3(512), 0, st, x, M, K, w, N, S, part,
                      out, mode, pf_krot, ng);
   return static_cast<int>(hipGetLastError());
@@ -484,6 +494,11 @@ static int launch_pf_cfg(int c, int tiles, hipStream_t st, const uint16_t* x, in
 template <int BM, int MTP, int LAG>
 static int launch_pf_grp(int tiles, hipStream_t st, const uint16_t* x, int M, int K, const uint16_t* w, int N, int S,
                          float* part, uint16_t* out, int mode, const PfGrp& grp) {
+  if (mode == PF_GLU) {
+    hipLaunchKernelGGL((gemm_pf_kernel<BM, MTP, false, 0, LAG, true, true>), dim3(tiles * S), dim3(512), 0, st, x, M, K, w,
+                       N, S, part, out, mode, 0, grp);
+    return static_cast<int>(hipGetLastError());
+  }
   hipLaunchKernelGGL((gemm_pf_kernel<BM, MTP, false, 0, LAG, true>), dim3(tiles * S), dim3(512), 0, st, x, M, K, w, N,
                      S, part, out, mode, 0, grp);
   return static_cast<int>(hipGetLastError());
@@ -492,23 +507,24 @@ static int launch_pf_grp(int tiles, hipStream_t st, const uint16_t* x, int M, in
 // Grouped (MoE experts, moe_align layout): out / part rows are the P sorted rows; w is
 // [E, N, K]; rows gathers x (nullptr: x is already in sorted order); max_pairs bounds
 // the real rows over all experts (sizes the grid: sum over experts of ceil(segment / BM)
-// <= (max_pairs + 63 E) / BM + E). Lag-2 configs 6 / 7 / 8 only.
+// <= (max_pairs + 63 E) / BM + E). Lag-2 configs 6 / 7 / 8 only. top: rows[] counts
+// (token, choice) pairs; kind / limit / alpha: PF_GLU's activation (w [E, gate F | up F, K]).
 int gemm_pf_grouped(const uint16_t* x, const int32_t* rows, const int32_t* offs, int E, int P, int K,
                     const uint16_t* w, int N, int max_pairs, float* part, uint16_t* out, int S, int mode, int cfg,
-                    hipStream_t st) {
+                    hipStream_t st, int top, int kind, float limit, float alpha) {
   if (E < 1 || P < 1 || P % 64 || max_pairs < 1 || offs == nullptr || K < 64 || K % 64 || N < pf::BN ||
-      N % pf::BN || S < 1 || S > K / 64 || cfg < 6 || cfg > 8)
+      N % pf::BN || S < 1 || S > K / 64 || cfg < 6 || cfg > 8 || top < 1)
     return 1;
   if (mode == PF_PARTIAL) {
     if (part == nullptr) return 1;
-  } else if (mode == PF_BF16 || mode == PF_SILU) {
+  } else if (mode == PF_BF16 || mode == PF_SILU || (mode == PF_GLU && (kind == kGluGeluTanh || kind == kGluClamped))) {
     if (out == nullptr || S != 1) return 1;
   } else {
     return 1;
   }
   const int bm = pf_cfg_bm(cfg);
   const int mt = (max_pairs + 63 * E) / bm + E;
-  const PfGrp grp{rows, offs, E, mt, static_cast<int64_t>(N) * K};
+  const PfGrp grp{rows, offs, E, mt, static_cast<int64_t>(N) * K, top, kind, limit, alpha};
   const int tiles = mt * (N / pf::BN);
   switch (cfg) {
     case 6: return launch_pf_grp<288, 3, 2>(tiles, st, x, P, K, w, N, S, part, out, mode, grp);

@@ -28,7 +28,7 @@ int gemm_m64g_ar(const uint16_t*, int, int, const uint16_t*, int, float*, int, i
                  const void*, hipStream_t);
 int m64g_ar_desc_bytes();
 int gemm_pf_grouped(const uint16_t*, const int32_t*, const int32_t*, int, int, int, const uint16_t*, int, int, float*,
-                    uint16_t*, int, int, int, hipStream_t);
+                    uint16_t*, int, int, int, hipStream_t, int, int, float, float);
 int gemm_pf(const uint16_t*, int, int, const uint16_t*, int, float*, uint16_t*, int, int, int, hipStream_t);
 void set_pf_krot(int);
 void set_k_rotation(int mode);
@@ -284,7 +284,7 @@ PYBIND11_MODULE(_kernels, m) {
                               int max_pairs, uintptr_t part, uintptr_t out, int splits, int mode, int cfg,
                               uintptr_t st) {
     check(xgk::gemm_pf_grouped(P<uint16_t>(x), P<int32_t>(rows), P<int32_t>(offs), E, n_rows, K, P<uint16_t>(w), N,
-                               max_pairs, P<float>(part), P<uint16_t>(out), splits, mode, cfg, S(st)),
+                               max_pairs, P<float>(part), P<uint16_t>(out), splits, mode, cfg, S(st), 1, 0, 0.f, 0.f),
           "gemm_pf_grouped");
   });
   m.def("set_pf_krot", [](int on) { xgk::set_pf_krot(on); });

@@ -14,7 +14,8 @@
 //                    read (the waves then repeat the same selection, so every barrier is met by all of them).
 //                    gate != nullptr: a logit after the experts' ones, gate[t] = sigmoid(it), takes no part in the
 //                    routing (the gate of an expert that runs for every token).
-//   moe_align        (token, choice) pairs sorted by expert into tiles of `tm` rows (padded with -1)
+//   moe_align        (token, choice) pairs sorted by expert into tiles of `tm` rows (padded with -1); offs: the experts'
+//                    padded starts [E + 1] (what gemm_pf's grouped form walks)
 //   grouped_gemm     per tile: rows x expert weights, in one of three modes:
 //                      kGemmRows    A rows as they lie in the sorted layout -> fp32 rows (the second product)
 //                      kGemmGated   A rows gathered by token; weights [gate | up]; output glu(gate, up)
@@ -25,29 +26,23 @@
 //                    nullptr = 1)
 //
 // Activations / weights are T = float or bf16; router, weights of the sum and the sum itself are fp32.
+#include "glu.h"
 #include "mixers_common.h"
 
 #include <algorithm>
 
 namespace xgm {
 
-constexpr int kGluGeluTanh = 0, kGluClamped = 1, kActRelu2 = 2;
+using xgk::glu;
+using xgk::kGluClamped;
+using xgk::kGluGeluTanh;
+constexpr int kActRelu2 = 2;
 constexpr int kGemmRows = 0, kGemmGated = 1, kGemmAct = 2;
 
 __device__ __forceinline__ float act1(int kind, float z) {
   (void)kind;  // kActRelu2
   const float r = fmaxf(z, 0.f);
   return r * r;
-}
-
-__device__ __forceinline__ float glu(int kind, float g, float u, float limit, float alpha) {
-  if (kind == kGluGeluTanh) {
-    const float c = 0.7978845608028654f;  // sqrt(2 / pi)
-    return 0.5f * g * (1.f + tanhf(c * (g + 0.044715f * g * g * g))) * u;
-  }
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g * sigmoidf(alpha * g) * (u + 1.f);
 }
 
 template <typename T>
@@ -216,7 +211,8 @@ __global__ __launch_bounds__(256) void grouped_router_kernel(const float* __rest
 // ------------------------------------------------------------------ pairs -> expert tiles (one workgroup)
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restrict__ ids, int pairs, int E, int cap,
                                                          int kTileM, int32_t* __restrict__ rows,
-                                                         int32_t* __restrict__ tile_expert, int32_t* __restrict__ dest) {
+                                                         int32_t* __restrict__ tile_expert, int32_t* __restrict__ dest,
+                                                         int32_t* __restrict__ offs) {
   extern __shared__ int si[];
   int* cnt = si;          // [E]
   int* off = si + E;      // [E + 1] padded starts
@@ -238,6 +234,10 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int32_t* __restri
   for (int e = threadIdx.x; e < E; e += blockDim.x) {
     for (int tl = off[e] / kTileM; tl < off[e + 1] / kTileM; ++tl) tile_expert[tl] = e;
     cnt[e] = 0;  // becomes the fill cursor
+    if (offs) {
+      offs[e] = off[e];
+      if (e == E - 1) offs[E] = off[E];
+    }
   }
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
@@ -618,10 +618,11 @@ int grouped_router(const float* logits, const float* corr, int T_, int E, int co
 }
 
 int moe_align(const int32_t* ids, int pairs, int E, int cap, int tm, int32_t* rows, int32_t* tile_expert, int32_t* dest,
-              hipStream_t st) {
+              int32_t* offs, hipStream_t st) {
   if (pairs <= 0) return 0;
   if (E < 1 || E > 4096 || tm < 16 || tm % 16 != 0 || cap % tm != 0 || cap < pairs + E * (tm - 1)) return -1;
-  moe_align_kernel<<<1, 1024, (2 * E + 1) * sizeof(int), st>>>(ids, pairs, E, cap, tm, rows, tile_expert, dest);
+  moe_align_kernel<<<1, 1024, (2 * E + 1) * sizeof(int), st>>>(ids, pairs, E, cap, tm, rows, tile_expert, dest,
+                                                                   offs);
   return 0;
 }
 

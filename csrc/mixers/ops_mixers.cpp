@@ -9,6 +9,10 @@
 
 namespace py = pybind11;
 
+namespace xgk {
+int gemm_pf_grouped(const uint16_t*, const int32_t*, const int32_t*, int, int, int, const uint16_t*, int, int, float*,
+                    uint16_t*, int, int, int, hipStream_t, int, int, float, float);
+}
 namespace xgm {
 void embed_rows(const int32_t*, const void*, bool, float*, int, int, int, const void*, const int32_t*, int, float,
                 hipStream_t);
@@ -54,7 +58,7 @@ int hyper_residual(const float*, bool, float*, int, const void*, int64_t, bool, 
                    const float*, int, const float*, const float*, const float*, const float*, float, float*, void*, bool,
                    int, int, hipStream_t);
 void soft_cap(void*, bool, float, int64_t, hipStream_t);
-int moe_align(const int32_t*, int, int, int, int, int32_t*, int32_t*, int32_t*, hipStream_t);
+int moe_align(const int32_t*, int, int, int, int, int32_t*, int32_t*, int32_t*, int32_t*, hipStream_t);
 int grouped_gemm(const void*, bool, int64_t, const void*, const int32_t*, const int32_t*, int, int, int, int, int, int, void*,
                  int, float, float, const float*, bool, hipStream_t);
 int mingru_scan(const void*, bool, int64_t, int, int, int, int, const float*, const float*, float*, const int32_t*,
@@ -287,9 +291,9 @@ PYBIND11_MODULE(_mixers, m) {
     check(rc, "grouped_router");
   });
   m.def("moe_align", [](uintptr_t ids, int pairs, int E, int cap, int tm, uintptr_t rows, uintptr_t tile_expert,
-                        uintptr_t dest, uintptr_t st) {
+                        uintptr_t dest, uintptr_t offs, uintptr_t st) {
     int rc = xgm::moe_align(P<const int32_t>(ids), pairs, E, cap, tm, P<int32_t>(rows), P<int32_t>(tile_expert),
-                            P<int32_t>(dest), S(st));
+                            P<int32_t>(dest), P<int32_t>(offs), S(st));
     check(rc, "moe_align");
   });
   m.def("grouped_gemm", [](uintptr_t A, bool f32, int64_t lda, uintptr_t Wt, uintptr_t rows, uintptr_t tile_expert, int cap,
@@ -300,6 +304,16 @@ PYBIND11_MODULE(_mixers, m) {
                                P<const int32_t>(tile_expert), cap, tm, top, Nout, K, mode, P<void>(out), kind, limit, alpha,
                                P<const float>(row_scale), mfma, S(st));
     check(rc, "grouped_gemm");
+  });
+  // prompt-sized expert products on gemm_pf's grouped form (csrc/kernels/gemm_pf.hip): mode 3 = gated epilogue on
+  // [gate | up] weights, rows gathered by rows[] / top; mode 1 = fp32 rows of the sorted layout
+  m.def("gemm_pf_grouped", [](uintptr_t x, uintptr_t rows, uintptr_t offs, int E, int n_rows, int K, uintptr_t w, int N,
+                              int max_pairs, uintptr_t part, uintptr_t out, int mode, int cfg, int top, int kind,
+                              float limit, float alpha, uintptr_t st) {
+    int rc = xgk::gemm_pf_grouped(P<const uint16_t>(x), P<const int32_t>(rows), P<const int32_t>(offs), E, n_rows, K,
+                                  P<const uint16_t>(w), N, max_pairs, P<float>(part), P<uint16_t>(out), 1, mode, cfg, S(st),
+                                  top, kind, limit, alpha);
+    check(rc, "gemm_pf_grouped");
   });
   m.def("moe_combine", [](uintptr_t y, uintptr_t dest, uintptr_t wts, int T, int top, int W, uintptr_t out, uintptr_t st) {
     xgm::moe_combine(P<const float>(y), P<const int32_t>(dest), P<const float>(wts), T, top, W, P<float>(out), S(st));

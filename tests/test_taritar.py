@@ -576,7 +576,8 @@ def test_clamped_gate_of_dense_layers(device, dtype, T, ff, limit):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("T,E,top,K,F_", [(7, 5, 2, 40, 24), (50, 1, 1, 32, 16), (100, 1, 1, 64, 32), (300, 3, 3, 64, 48),
-                                          (700, 4, 1, 96, 64), (1300, 4, 2, 128, 32), (64, 12, 1, 24, 10)])
+                                          (700, 4, 1, 96, 64), (1300, 4, 2, 128, 32), (64, 12, 1, 24, 10),
+                                          (900, 4, 2, 256, 128), (300, 3, 3, 256, 256), (2100, 5, 1, 512, 384)])
 def test_routed_experts_with_a_clamped_gate(device, dtype, T, E, top, K, F_):
     """Every grouped-GEMM path; softmax weights at the output; the sum over choices inside the residual write."""
     dt = getattr(torch, dtype)

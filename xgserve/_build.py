@@ -133,9 +133,10 @@ def build_kernels(force: bool = False, jobs: int = 8, probes: bool = False) -> P
 
 
 def build_mixers(force: bool = False, jobs: int = 8) -> Path:
-    srcs = sorted((CSRC / "mixers").glob("*.hip"))
+    # (gemm_pf: the prompt-sized expert products, the same source as in the kernel library)
+    srcs = sorted((CSRC / "mixers").glob("*.hip")) + [CSRC / "kernels" / "gemm_pf.hip"]
     cpp = sorted((CSRC / "mixers").glob("*.cpp"))
-    hdrs = [CSRC / "kernels" / "common.h"] + sorted((CSRC / "mixers").glob("*.h"))
+    hdrs = [CSRC / "kernels" / h for h in ("common.h", "glds.h", "glu.h")] + sorted((CSRC / "mixers").glob("*.h"))
     out = PKG / f"_mixers{EXT}"
     flags = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-fvisibility=hidden", "-Wno-unused-result",
              *NO_PK_F32]

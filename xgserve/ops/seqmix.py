@@ -20,6 +20,7 @@ import torch
 
 from .. import tune
 from ._native import is_f32, mixers, native_device, stream_ptr
+from .moe import _moe_pf_cfg
 
 
 @dataclass
@@ -752,6 +753,9 @@ GLU_GELU_TANH, GLU_CLAMPED = 0, 1
 ACT_RELU2 = 2   # routed_experts(kind=...): an expert without a gate, W_down relu(W_up h)^2
 # XGS_TUNE moe_mfma=0: the general grouped GEMM for bf16 too (A/B and tests)
 MOE_MFMA = tune.get_bool("moe_mfma", True)
+# XGS_TUNE seq_moe_pf=0: the gated experts of long steps stay on the tiles of csrc/mixers (A/B and tests)
+SEQ_MOE_PF = tune.get_bool("seq_moe_pf", True)
+MOE_PF_MIN = 96   # average rows per expert from which gated experts run on gemm_pf's grouped form
 MOE_TILE_SMALL, MOE_TILES_BIG = 16, (128, 64, 32)   # rows per expert tile of the sorted layout
 MOE_TILE32_MIN = 12   # average rows per expert from which 32-row tiles replace 16-row ones (XGS_TUNE moe_tile32_min)
 MOE_TILE32_MIN = tune.get_int("moe_tile32_min", MOE_TILE32_MIN)
@@ -885,23 +889,40 @@ def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: to
     # rows of an expert are padded to whole tiles: 128 / 64-row tiles once the average expert has that many; 32-row
     # tiles once many experts would need a second 16-row tile (their weights would be streamed twice); else 16
     tm = next((t for t in MOE_TILES_BIG if pairs >= (t if t > 32 else MOE_TILE32_MIN) * E), MOE_TILE_SMALL)
+    # ... or run on gemm_pf's grouped form: both operands by LDS DMA, 64-row segments, 256-column tiles
+    pf = SEQ_MOE_PF and MOE_MFMA and gated and h.dtype == torch.bfloat16 and pairs >= MOE_PF_MIN * E and K % 64 == 0 \
+        and F_ % 128 == 0 and W % 256 == 0
+    if pf:
+        tm = 64
     cap = (pairs + E * (tm - 1) + tm - 1) // tm * tm
     dev = h.device
-    meta = torch.empty(cap + cap // tm + pairs, dtype=torch.int32, device=dev)
-    rows, tile_e, dest = meta[:cap], meta[cap:cap + cap // tm], meta[cap + cap // tm:]
-    M.moe_align(_i32(ids).data_ptr(), pairs, E, cap, tm, rows.data_ptr(), tile_e.data_ptr(), dest.data_ptr(), stream_ptr())
+    meta = torch.empty(cap + cap // tm + pairs + E + 1, dtype=torch.int32, device=dev)
+    rows, tile_e, dest, offs = meta.split((cap, cap // tm, pairs, E + 1))
+    M.moe_align(_i32(ids).data_ptr(), pairs, E, cap, tm, rows.data_ptr(), tile_e.data_ptr(), dest.data_ptr(),
+                offs.data_ptr(), stream_ptr())
     act = torch.empty(cap, F_, dtype=h.dtype, device=dev)
+    if pf:
+        cfg = _moe_pf_cfg(pairs, E)
+        y = torch.empty(cap, W, dtype=torch.float32, device=dev)
+        M.gemm_pf_grouped(h.data_ptr(), rows.data_ptr(), offs.data_ptr(), E, cap, K, w13.data_ptr(), 2 * F_, pairs, 0,
+                          act.data_ptr(), 3, cfg, top, int(kind), float(limit), float(alpha), stream_ptr())
+        M.gemm_pf_grouped(act.data_ptr(), 0, offs.data_ptr(), E, cap, F_, w2.data_ptr(), W, pairs, y.data_ptr(), 0, 1, cfg,
+                          1, 0, 0.0, 0.0, stream_ptr())
+        return _routed_sum(M, y, dest, None if scale_input else wts, T, top, W, combine)
     M.grouped_gemm(h.data_ptr(), is_f32(h), h.stride(0), w13.data_ptr(), rows.data_ptr(), tile_e.data_ptr(), cap, tm, top,
                    F_, K, 1 if gated else 2, act.data_ptr(), int(kind), float(limit), float(alpha),
                    wts.data_ptr() if scale_input else 0, MOE_MFMA, stream_ptr())
     y = torch.empty(cap, W, dtype=torch.float32, device=dev)
     M.grouped_gemm(act.data_ptr(), is_f32(act), F_, w2.data_ptr(), rows.data_ptr(), tile_e.data_ptr(), cap, tm, top, W, F_,
                    0, y.data_ptr(), 0, 0.0, 0.0, 0, MOE_MFMA, stream_ptr())
+    return _routed_sum(M, y, dest, None if scale_input else wts, T, top, W, combine)
+
+
+def _routed_sum(M, y, dest, wts, T, top, W, combine):
     if not combine:
-        return RoutedRows(y, dest.view(T, top), None if scale_input else wts)
-    out = torch.empty(T, W, dtype=torch.float32, device=dev)
-    M.moe_combine(y.data_ptr(), dest.data_ptr(), 0 if scale_input else wts.data_ptr(), T, top, W, out.data_ptr(),
-                  stream_ptr())
+        return RoutedRows(y, dest.view(T, top), wts)
+    out = torch.empty(T, W, dtype=torch.float32, device=y.device)
+    M.moe_combine(y.data_ptr(), dest.data_ptr(), _p(wts), T, top, W, out.data_ptr(), stream_ptr())
     return out
 
 
