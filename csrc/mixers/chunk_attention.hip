@@ -30,23 +30,9 @@
 //                     q to a dense tensor, k / v to the cache rows slot_mapping[t]
 //
 // Activations / caches are T = float or bf16; norms, scores, probabilities and the accumulators are fp32.
-#include "mixers_common.h"
+#include "attention_common.h"
 
 namespace xgm {
-
-constexpr int kMaskCausal = 0, kMaskWindow = 1, kMaskChunk = 2;
-constexpr int kValuesOwn = -1, kValuesAll = -2;
-constexpr int kWeightsSoftmax = 0, kWeightsSigmoid = 1;
-// matrix-core forms of the bounded softmax: kWeightsBounded needs no running maximum (|score| <= softcap, so every
-// exponential and every sum of them stays in range without a reference), kWeightsCapped keeps one (large bounds, sinks)
-constexpr int kWeightsBounded = 2, kWeightsCapped = 3;
-constexpr float kBoundedMaxLog2 = 90.f;   // largest bound in units of ln 2: 2^90 x 2^20 keys x values stays far from 2^127
-
-__device__ __forceinline__ int first_visible(int mask, int size, int pos) {
-  if (mask == kMaskWindow) return max(0, pos - size + 1);
-  if (mask == kMaskChunk) return (pos / size) * size;
-  return 0;
-}
 
 // ------------------------------------------------------------------ projections -> normed q, cache rows
 template <typename T>
@@ -215,22 +201,6 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
 // operand (V^T) is a transposed LDS read of the staged V rows.
 constexpr int kKT = 64;
 
-__device__ __forceinline__ float exp2_fast(float x) {
-#if defined(__HIP_DEVICE_COMPILE__)
-  return __builtin_amdgcn_exp2f(x);
-#else
-  return exp2f(x);
-#endif
-}
-
-__device__ __forceinline__ float rcp_fast(float x) {
-#if defined(__HIP_DEVICE_COMPILE__)
-  return __builtin_amdgcn_rcpf(x);
-#else
-  return 1.f / x;
-#endif
-}
-
 template <int NKK_MAX, int NMT_MAX, int NW, int WFN>
 __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ kcache, const bf16* __restrict__ vcache,
@@ -303,7 +273,6 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
     qf[kk] = xgk::as_frag(v);
   }
   // scores are kept in units of ln 2 (exp2 is one instruction): score * log2(e)
-  constexpr float kLog2e = 1.4426950408889634f;
   constexpr bool capped = WFN == kWeightsBounded || WFN == kWeightsCapped, bounded = WFN == kWeightsBounded;
   // bounded scores: c tanh(z / c) = c - 2 c / (1 + e^(2 z / c)), again with 2^x: the factor below gives the exponent
   const float cap2 = capped ? softcap * kLog2e : 0.f;
@@ -476,43 +445,37 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_mfma_kernel(
   }
 }
 
-// merge the key shares of a single-token step: out = sum_s 2^(m_s - M) o_s / sum_s 2^(m_s - M) l_s (m in units of ln 2)
-__global__ void masked_attention_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
-                                                const int32_t* __restrict__ slots, bf16* __restrict__ out, int Ttot, int H,
-                                                int dv, int nsplit, const bf16* __restrict__ gate, int64_t ld_gate,
-                                                int gate_elem, int wfn) {
-  const int t = blockIdx.x, h = blockIdx.y;
+// merge the key shares of a single-token step: out = sum_s 2^(m_s - M) o_s / sum_s 2^(m_s - M) l_s (m in units of ln 2);
+// unnormalised weights: the shares simply add up. At most 64 shares: lane s of every wave holds share s's factor.
+__global__ __launch_bounds__(256) void masked_attention_combine_kernel(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml, const int32_t* __restrict__ slots,
+    bf16* __restrict__ out, int Ttot, int H, int dv, int nsplit, const bf16* __restrict__ gate, int64_t ld_gate,
+    int gate_elem, int wfn) {
+  __shared__ float ws[64];
+  const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
   if (slots[t] < 0) return;  // single-token steps: row t is sequence t (its output row was zeroed)
-  if (wfn == kWeightsSigmoid) {   // unnormalised weights: the shares simply add up
-    const float gh = (gate && !gate_elem) ? sigmoidf(bf2f(gate[(int64_t)t * ld_gate + h])) : 1.f;
-    for (int d = threadIdx.x; d < dv; d += blockDim.x) {
-      float acc = 0.f;
-      for (int sp = 0; sp < nsplit; ++sp) acc += part_o[(((int64_t)sp * Ttot + t) * H + h) * dv + d];
-      if (gate && gate_elem) acc *= sigmoidf(bf2f(gate[(int64_t)t * ld_gate + (int64_t)h * dv + d]));
-      out[((int64_t)t * H + h) * dv + d] = f2bf(acc * gh);
-    }
-    return;
+  const int64_t step = (int64_t)Ttot * H, row0 = (int64_t)t * H + h;
+  float w = lane < nsplit ? 1.f : 0.f, inv = 1.f;
+  if (wfn != kWeightsSigmoid) {
+    const float ms = lane < nsplit ? part_ml[2 * (row0 + lane * step)] : -INFINITY;
+    const float ls = lane < nsplit ? part_ml[2 * (row0 + lane * step) + 1] : 0.f;
+    const float M = wave_max(ms);
+    w = ms == -INFINITY ? 0.f : exp2_fast(ms - M);
+    const float L = wave_sum(w * ls);
+    inv = L > 0.f ? 1.f / L : 0.f;
   }
-  float M = -INFINITY;
-  for (int sp = 0; sp < nsplit; ++sp) M = fmaxf(M, part_ml[2 * (((int64_t)sp * Ttot + t) * H + h)]);
-  float L = 0.f;
-  for (int sp = 0; sp < nsplit; ++sp) {
-    const int64_t row = ((int64_t)sp * Ttot + t) * H + h;
-    const float ms = part_ml[2 * row];
-    if (ms != -INFINITY) L += exp2_fast(ms - M) * part_ml[2 * row + 1];
-  }
-  float inv = L > 0.f ? 1.f / L : 0.f;
+  if (threadIdx.x < 64) ws[lane] = w;
+  __syncthreads();
   if (gate && !gate_elem) inv *= sigmoidf(bf2f(gate[(int64_t)t * ld_gate + h]));
   for (int d = threadIdx.x; d < dv; d += blockDim.x) {
     float acc = 0.f;
-    for (int sp = 0; sp < nsplit; ++sp) {
-      const int64_t row = ((int64_t)sp * Ttot + t) * H + h;
-      const float ms = part_ml[2 * row];
-      if (ms != -INFINITY) acc += exp2_fast(ms - M) * part_o[row * dv + d];
+#pragma unroll 8
+    for (int sp = 0; sp < nsplit; ++sp) {   // (a share without keys holds zeros)
+      acc += ws[sp] * part_o[(row0 + sp * step) * dv + d];
     }
     acc *= inv;
     if (gate && gate_elem) acc *= sigmoidf(bf2f(gate[(int64_t)t * ld_gate + (int64_t)h * dv + d]));
-    out[((int64_t)t * H + h) * dv + d] = f2bf(acc);
+    out[row0 * dv + d] = f2bf(acc);
   }
 }
 
@@ -868,7 +831,7 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
       (gate_elem && vmode != kValuesOwn) || wfn < 0 || wfn > 1 || (wfn == kWeightsSigmoid && (sink || softcap > 0.f)) ||
       keep < 0 || (keep > 0 && mask != kMaskWindow))
     return -1;
-  if (softcap > 0.f) wfn = (softcap * 1.4426950408889634f <= kBoundedMaxLog2 && !sink && !r1) ? kWeightsBounded : kWeightsCapped;
+  if (softcap > 0.f) wfn = (softcap * kLog2e <= kBoundedMaxLog2 && !sink && !r1) ? kWeightsBounded : kWeightsCapped;
   const int ge = gate_elem ? 1 : 0;
   const int rep = H / G;
   const int RH = rep >= 4 ? 4 : rep >= 2 ? 2 : 1;
@@ -881,8 +844,20 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
   if (!head_slots && (nw_hint == 4 || nw_hint == 8 || (nw_hint == 16 && dv <= 128))) nw = nw_hint;
   const int tpb = nw / RH;
   dim3 grid((max_q + 16 * tpb - 1) / (16 * tpb), G * ((rep + RH - 1) / RH), ns);
+  if (nsplit > 64) return -4;
   if (!head_slots || nsplit < 1 || (nsplit > 1 && (!part_o || !part_ml))) nsplit = 1;
   if (head_slots) grid = dim3(nsplit, G, ns);
+  if (head_slots) {
+    const AttnArgs args{(const bf16*)q, (const bf16*)kcache, (const bf16*)vcache, block_tables, bt_width, bs, qsl, seq_lens,
+                        slots, temp, sink, (bf16*)out, T_, ns, H, G, dk, dv_head, mask, size, scale, (const bf16*)gate,
+                        ld_gate, r1, r2, vmode, ge, hbias, softcap, keep};
+    if (single_attention(args, wfn, nsplit, part_o, part_ml, st)) {
+      if (nsplit > 1)
+        masked_attention_combine_kernel<<<dim3(T_, H), dv > 64 ? 128 : 64, 0, st>>>(part_o, part_ml, slots, (bf16*)out, T_, H, dv, nsplit,
+                                                                    (const bf16*)gate, ld_gate, ge, wfn);
+      return 0;
+    }
+  }
   const size_t lds = (size_t)kKT * (dk + 8 + dv + 8) * sizeof(uint16_t);
 #define XGM_MK2(NKK, NMT, NW, WFN)                                                                                    \
   masked_attention_mfma_kernel<NKK, NMT, NW, WFN><<<grid, 64 * NW, lds, st>>>(                                        \
@@ -908,7 +883,7 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
     XGM_MK(NKK, NMT, 4)                                                                                               \
   }                                                                                                                   \
   if (nsplit > 1)                                                                                                     \
-    masked_attention_combine_kernel<<<dim3(T_, H), 64, 0, st>>>(part_o, part_ml, slots, (bf16*)out, T_, H, dv, nsplit, \
+    masked_attention_combine_kernel<<<dim3(T_, H), dv > 64 ? 128 : 64, 0, st>>>(part_o, part_ml, slots, (bf16*)out, T_, H, dv, nsplit, \
                                                                 (const bf16*)gate, ld_gate, ge, wfn);                 \
   return 0;
   if (dk <= 64 && dv <= 64) { XGM_MM(2, 4) }

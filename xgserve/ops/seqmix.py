@@ -539,8 +539,8 @@ MASK_CAUSAL, MASK_WINDOW, MASK_CHUNK = 0, 1, 2
 ATTN_MFMA = tune.get_bool("attn_mfma", True)
 # XGS_TUNE attn_waves=4|8|16: waves per workgroup of the matrix-core kernel on prompt portions (0: by portion length)
 ATTN_WAVES = tune.get_int("attn_waves", 0)
-ATTN_MAX_SPLITS = 8      # key shares per single-token row, at most
-ATTN_SPLIT_WGS = 2048    # ... while the launch stays under about this many workgroups
+ATTN_MAX_SPLITS = 32     # key shares per single-token row, at most (64 in the merging kernel)
+ATTN_SPLIT_WGS = 512     # ... while the launch stays under about this many workgroups (measured: 2 per compute unit)
 
 
 def first_visible(mask: int, size: int, pos: int) -> int:
