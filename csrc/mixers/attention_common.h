@@ -61,4 +61,9 @@ constexpr int kSingleMaxRep = 16;   // query heads per key / value head the sing
 // unnormalised shares go to part_o / part_ml. Returns false when the sizes are not served.
 bool single_attention(const AttnArgs& a, int wfn, int nsplit, float* part_o, float* part_ml, hipStream_t st);
 
+// prompt_attention.hip: portions of more than kPromptMinRows rows (dk and dv 64 or 128, block sizes a multiple of 16).
+// Returns false when the sizes are not served.
+constexpr int kPromptMinRows = 32;
+bool prompt_attention(const AttnArgs& a, int max_q, int wfn, hipStream_t st);
+
 }  // namespace xgm

@@ -847,11 +847,12 @@ int masked_attention_mfma(const void* q, const void* kcache, const void* vcache,
   if (nsplit > 64) return -4;
   if (!head_slots || nsplit < 1 || (nsplit > 1 && (!part_o || !part_ml))) nsplit = 1;
   if (head_slots) grid = dim3(nsplit, G, ns);
-  if (head_slots) {
+  {
     const AttnArgs args{(const bf16*)q, (const bf16*)kcache, (const bf16*)vcache, block_tables, bt_width, bs, qsl, seq_lens,
                         slots, temp, sink, (bf16*)out, T_, ns, H, G, dk, dv_head, mask, size, scale, (const bf16*)gate,
                         ld_gate, r1, r2, vmode, ge, hbias, softcap, keep};
-    if (single_attention(args, wfn, nsplit, part_o, part_ml, st)) {
+    if (!head_slots && max_q > kPromptMinRows && nw_hint == 0 && prompt_attention(args, max_q, wfn, st)) return 0;
+    if (head_slots && single_attention(args, wfn, nsplit, part_o, part_ml, st)) {
       if (nsplit > 1)
         masked_attention_combine_kernel<<<dim3(T_, H), dv > 64 ? 128 : 64, 0, st>>>(part_o, part_ml, slots, (bf16*)out, T_, H, dv, nsplit,
                                                                     (const bf16*)gate, ld_gate, ge, wfn);

@@ -420,7 +420,7 @@ def _attention_case(device, dtype, H, G, dk, dv, bs, T, single, mask, cap, stron
 
 
 ATTN_TOL = {"float32": 1e-4, "bfloat16": 4e-2}
-SHAPES = [(6, 2, 20, 12), (1, 1, 32, 32), (8, 2, 64, 32), (4, 4, 96, 48), (16, 2, 32, 128), (20, 1, 64, 64), (4, 2, 128, 128)]
+SHAPES = [(6, 2, 20, 12), (1, 1, 32, 32), (8, 2, 64, 32), (4, 4, 96, 48), (16, 2, 32, 128), (20, 1, 64, 64), (4, 2, 128, 128), (3, 3, 64, 128), (6, 3, 128, 64)]
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
@@ -430,7 +430,8 @@ SHAPES = [(6, 2, 20, 12), (1, 1, 32, 32), (8, 2, 64, 32), (4, 4, 96, 48), (16, 2
 def test_bounded_scores_in_windows_with_kept_tokens(device, dtype, shape, single, size, keep, cap):
     """For the general and the matrix-core kernels, as a prompt portion and as single tokens: windows and kept runs shorter
     and longer than a key tile, bounds narrow (no running maximum) and wide (with one), none, and no window at all."""
-    got, ref = _attention_case(device, dtype, *shape, bs=4, T=140, single=single, cap=cap,
+    bs = 16 if min(shape[2:]) >= 64 else 4
+    got, ref = _attention_case(device, dtype, *shape, bs=bs, T=140, single=single, cap=cap,
                                mask={"size": size, "keep_first": keep} if size else None,
                                rot={"base": 50.0, "dims": shape[2] // 4 * 2})
     assert rel_err(got, ref) < ATTN_TOL[dtype]
@@ -440,14 +441,14 @@ def test_bounded_scores_in_windows_with_kept_tokens(device, dtype, shape, single
 @pytest.mark.parametrize("size,keep", [(1, 0), (2, 5), (16, 16), (17, 1), (40, 64), (64, 4), (65, 66)])
 @pytest.mark.parametrize("edge", ["window-in", "window-out", "first", "kept-in", "kept-out", "self"])
 @pytest.mark.parametrize("single", [False, True], ids=["prompt", "decoded"])
-@pytest.mark.parametrize("dk", [32, 20])
-def test_one_standing_out_key_at_an_edge(device, dtype, size, keep, edge, single, dk):
+@pytest.mark.parametrize("dk,dv", [(32, 16), (20, 16), (64, 64), (128, 128)])
+def test_one_standing_out_key_at_an_edge(device, dtype, size, keep, edge, single, dk, dv):
     """The key that stands out for the last query is the oldest one of the window or the one before it, the first / last
     kept one or the one after it, or its own: a key lost, added or read from the wrong row moves the output."""
     T = 150
     j = {"window-in": T - size, "window-out": T - 1 - size, "first": 0, "kept-in": max(keep - 1, 0), "kept-out": keep,
          "self": T - 1}[edge]
-    got, ref = _attention_case(device, dtype, 4, 2, dk, 16, bs=16, T=T, single=single, cap=12.0,
+    got, ref = _attention_case(device, dtype, 4, 2, dk, dv, bs=16, T=T, single=single, cap=12.0,
                                mask={"size": size, "keep_first": keep}, strong=(T - 1, j), rot={"base": 500.0, "dims": 16})
     assert rel_err(got[-1:], ref[-1:]) < ATTN_TOL[dtype]
     assert rel_err(got, ref) < ATTN_TOL[dtype]
@@ -456,9 +457,10 @@ def test_one_standing_out_key_at_an_edge(device, dtype, size, keep, edge, single
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("back", [0, 1, 15, 16, 17, 63, 64, 127, 128, 130, 299, 300])
 @pytest.mark.parametrize("single", [False, True], ids=["prompt", "decoded"])
-def test_far_key_without_a_window(device, dtype, back, single):
+@pytest.mark.parametrize("dk,dv", [(32, 16), (64, 64)])
+def test_far_key_without_a_window(device, dtype, back, single, dk, dv):
     T = 301
-    got, ref = _attention_case(device, dtype, 4, 2, 32, 16, bs=16, T=T, single=single, cap=12.0, mask=None,
+    got, ref = _attention_case(device, dtype, 4, 2, dk, dv, bs=16, T=T, single=single, cap=12.0, mask=None,
                                strong=(T - 1, T - 1 - back), rot={"base": 1e4, "dims": 32})
     assert rel_err(got[-1:], ref[-1:]) < ATTN_TOL[dtype]
     assert rel_err(got, ref) < ATTN_TOL[dtype]
@@ -521,6 +523,39 @@ def test_batches_of_single_tokens_with_unequal_contexts(device, dtype, G, dk, dv
                 sc = cap * torch.tanh(sc / cap) if cap else sc
                 ref[h] = torch.softmax(sc, 0) @ v[vis, h // rep]
             assert rel_err(both[i].float().cpu().view(1, -1), ref.view(1, -1)) < ATTN_TOL[dtype], (i, size, keep, cap)
+
+
+@pytest.mark.parametrize("device,dtype", CASES[1:])
+@pytest.mark.parametrize("G,dk,dv,rep", [(2, 64, 64, 4), (1, 128, 128, 2), (2, 64, 128, 1), (1, 32, 16, 3)])
+def test_batches_of_unequal_portions(device, dtype, G, dk, dv, rep):
+    """Portions of 1 to 200 tokens on contexts of 0 to 300, a sequence without a slot among them, in one launch."""
+    H, bs, dt = G * rep, 16, getattr(torch, dtype)
+    g = torch.Generator().manual_seed(dk + rep)
+    seqs = [(0, 0, 70), (1, 300, 1), (-1, 5, 9), (2, 17, 200), (3, 250, 33), (4, 129, 2), (5, 0, 1)]
+    perm = torch.randperm(96, generator=g).tolist()
+    tables, at = [], 0
+    for _, c, n in seqs:
+        k = (c + n + bs - 1) // bs
+        tables.append(perm[at:at + k])
+        at += k
+    kc = torch.randn(96 * bs, G * dk, generator=g).to(dt).to(device)
+    vc = torch.randn(96 * bs, G * dv, generator=g).to(dt).to(device)
+    q = torch.randn(sum(n for _, _, n in seqs), H * dk, generator=g).to(dt).to(device)
+    for kind, size, keep, cap in ((sq.MASK_CAUSAL, 0, 0, 6.0), (sq.MASK_WINDOW, 50, 20, 6.0), (sq.MASK_WINDOW, 21, 100, 0.0),
+                                  (sq.MASK_WINDOW, 130, 3, 99.0)):
+        both = sq.masked_attention(q, kc, vc, H, G, dk, dv, kind, size, 0.3, None, None, bs, seq_meta(device, seqs, bs, tables),
+                                   softcap=cap, keep_first=keep)
+        m = {"scale": 0.3, "softcap": cap, "mask": {"size": size, "keep_first": keep} if size else None}
+        o = 0
+        for i, (slot, c, n) in enumerate(seqs):
+            rows = torch.tensor([tables[i][p // bs] * bs + p % bs for p in range(c + n)])
+            if slot >= 0:
+                k, v = kc.cpu()[rows].to(F64).view(-1, G, dk), vc.cpu()[rows].to(F64).view(-1, G, dv)
+                qq = torch.zeros(c + n, H, dk, dtype=F64)
+                qq[c:] = q[o:o + n].cpu().to(F64).view(n, H, dk)
+                ref = orc.attend(qq, k, v, m)[c:]
+                assert rel_err(both[o:o + n].float().cpu(), ref.reshape(n, -1)) < ATTN_TOL[dtype], (i, size, keep, cap)
+            o += n
 
 
 @pytest.mark.parametrize("device", OP_CASES)
