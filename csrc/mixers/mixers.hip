@@ -35,6 +35,23 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const TW* __r
   const bool ok = id >= 0 && id < V;
   const int p = pos_table ? positions[t] : -1;
   const bool pk = p >= 0 && p < P;
+  if ((W & 3) == 0) {   // (rows of whole quads; the tables' storage is aligned)
+    for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x) {
+      float v[4] = {0.f, 0.f, 0.f, 0.f}, u[4];
+      if (ok) {
+        ld4(table + (int64_t)id * W + c, v);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] *= scale;
+      }
+      if (pk) {
+        ld4(pos_table + (int64_t)p * W + c, u);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] += u[e];
+      }
+      st4(out + (int64_t)t * W + c, v);
+    }
+    return;
+  }
   for (int c = threadIdx.x; c < W; c += blockDim.x) {
     float v = ok ? ldf(table + (int64_t)id * W + c) * scale : 0.f;
     if (pk) v += ldf(pos_table + (int64_t)p * W + c);

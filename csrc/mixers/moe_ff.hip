@@ -10,7 +10,7 @@
 //                    `top` highest eligible selection scores win; weight = score * scale (the correction does not
 //                    enter it, no normalisation).
 //                    For steps of few rows the logits x . rw[e] (fp32 rows and router weights) are formed here
-//                    by a four-wave workgroup per token, eight experts per sweep over the row, instead of being
+//                    by a workgroup per token, 8 or 16 logits per sweep over the row, instead of being
 //                    read (the waves then repeat the same selection, so every barrier is met by all of them).
 //                    gate != nullptr: a logit after the experts' ones, gate[t] = sigmoid(it), takes no part in the
 //                    routing (the gate of an expert that runs for every token).
@@ -78,7 +78,7 @@ constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kRateTop2 = 0, kRateMax = 1;
 
 // kRouterSweep: logits per sweep over the row when they are formed here
 template <int kRouterSweep>
-__global__ __launch_bounds__(256) void grouped_router_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
+__global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
                                                              int E, int count, int keep, int top, float scale,
                                                              int32_t* __restrict__ ids, float* __restrict__ wts,
                                                              const float* __restrict__ x, const float* __restrict__ rw,
@@ -605,9 +605,10 @@ int grouped_router(const float* logits, const float* corr, int T_, int E, int co
       top > keep * (E / count) || score < 0 || score > 1 || rating < 0 || rating > 1)
     return -1;
   if ((x != nullptr) != (rw != nullptr) || (x && W < 1) || (!x && !logits)) return -2;
-  const int nth = x ? 256 : 64;
+  // logits formed here: one pass over the row (every weight row's load in flight at once)
+  const int nth = x ? std::min(1024, std::max(64, ((W & 3) ? W + 63 : W / 4 + 63) / 64 * 64)) : 64;
   const int EL = E + (gate ? 1 : 0);
-  const size_t lds = (E + EL + 2 * count + 4 * 16) * sizeof(float);
+  const size_t lds = (E + EL + 2 * count + 16 * 16) * sizeof(float);
   if (x && EL > 8 && EL <= 16)
     grouped_router_kernel<16><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score,
                                                     rating, gate);

@@ -785,8 +785,8 @@ def glu_act(x: torch.Tensor, kind: int, limit: float = 0.0, alpha: float = 1.702
 
 
 ROUTER_FUSED_MAX_ROWS = 256     # steps of up to this many rows form the router logits inside the router kernel ...
-ROUTER_FUSED_MAX_WORK = 16384   # ... when experts x width stays within this (measured on 64 rows: 13 against 16 us at
-                                # 8 x 2048, 20 against 16 us at 8 x 4096)
+ROUTER_FUSED_MAX_LOGITS = 16    # ... while one sweep over the row forms them all (measured on 1 - 256 rows: 10 against 12 us
+                                # at 9 x 2048, 13 against 15 us at 9 x 4096; 13 - 18 against 12 - 15 us for 17 logits)
 
 
 SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1   # grouped_router(score=...)
@@ -809,7 +809,7 @@ def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Te
     if logits is None:
         assert rows.dtype == router_w.dtype == torch.float32 and rows.shape[1] == router_w.shape[1]
         fused = native_device(rows) and rows.shape[0] <= ROUTER_FUSED_MAX_ROWS and rows.is_contiguous() \
-            and router_w.is_contiguous() and router_w.numel() <= ROUTER_FUSED_MAX_WORK
+            and router_w.is_contiguous() and router_w.shape[0] <= ROUTER_FUSED_MAX_LOGITS
         if not fused:
             logits = torch.nn.functional.linear(rows, router_w)
     T, E = (rows.shape[0], router_w.shape[0]) if fused else logits.shape
