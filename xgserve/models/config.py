@@ -520,7 +520,8 @@ def from_hf_config(path: str, name: Optional[str] = None) -> ModelConfig:
                               c["norm"]["eps"], int(c["norm"].get("groups", 1)), int(c.get("max_position", 131072)))
     if c.get("architecture") == "Taritar":
         return taritar_config(name or "taritar", c["width"], c["vocab"], c["layers"], int(c["streams"]),
-                              c["embedding"]["scale"], c["norm"]["eps"], c.get("logit_softcap"), int(c["max_positions"]))
+                              c["embedding"]["scale"], c["norm"]["eps"], c.get("logit_softcap"),
+                              int(c.get("max_positions", 4096)))
     mt = c.get("model_type", "llama")
     eos = c.get("eos_token_id", 2)
     eos = eos if isinstance(eos, list) else [eos]

@@ -35,7 +35,11 @@ def model_class(cfg: ModelConfig):
 
 def _resolve_shapes(cfg: ModelConfig, checkpoint: str) -> None:
     """Sizes that only a tensor's shape gives (Dofivik: the rank of the decay projection; Loluzen: the taps of
-    a short convolution when the configuration leaves them out; Lotelix: the rank of the decay projection)."""
+    a short convolution when the configuration leaves them out; Lotelix: the rank of the decay projection;
+    Taritar: the number of learned positions)."""
+    if cfg.arch == "taritar":
+        cfg.max_position = int(_Reader(checkpoint).shape("pos")[0])
+        return
     if cfg.arch == "lotelix":
         r = _Reader(checkpoint)
         for i, spec in enumerate(cfg.layer_specs):
