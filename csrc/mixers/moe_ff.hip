@@ -10,8 +10,8 @@
 //                    `top` highest eligible selection scores win; weight = score * scale (the correction does not
 //                    enter it, no normalisation).
 //                    For steps of few rows the logits x . rw[e] (fp32 rows and router weights) are formed here
-//                    by a workgroup per token, 8 or 16 logits per sweep over the row, instead of being
-//                    read (the waves then repeat the same selection, so every barrier is met by all of them).
+//                    by a workgroup per token, 8, 12 or 16 logits per sweep over the row, instead of being
+//                    read; its first wave then selects.
 //                    gate != nullptr: a logit after the experts' ones, gate[t] = sigmoid(it), takes no part in the
 //                    routing (the gate of an expert that runs for every token).
 //   moe_align        (token, choice) pairs sorted by expert into tiles of `tm` rows (padded with -1); offs: the experts'
@@ -74,6 +74,14 @@ __global__ __launch_bounds__(256) void glu_act4_kernel(const T* __restrict__ in,
 // ------------------------------------------------------------------ router: one wave per token
 constexpr int kMaxEPL = 8;  // experts per lane: E <= 512
 
+// LDS hand-over between the lanes of one wave
+__device__ __forceinline__ void wave_sync() {
+  asm volatile("" ::: "memory");
+#if defined(__HIP_DEVICE_COMPILE__)
+  __builtin_amdgcn_wave_barrier();
+#endif
+}
+
 constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kRateTop2 = 0, kRateMax = 1;
 
 // kRouterSweep: logits per sweep over the row when they are formed here
@@ -101,15 +109,13 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
       for (int j = 0; j < kRouterSweep; ++j) acc[j] = 0.f;
       if (vec) {
         for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x) {
-          float a[4];
+          float a[4], b[kRouterSweep][4];   // (rows past the last repeat it: every load is issued before the first use)
           ld4(xr + c, a);
 #pragma unroll
+          for (int j = 0; j < kRouterSweep; ++j) ld4(rw + (int64_t)min(e0 + j, EL - 1) * W + c, b[j]);
+#pragma unroll
           for (int j = 0; j < kRouterSweep; ++j)
-            if (e0 + j < EL) {
-              float b[4];
-              ld4(rw + (int64_t)(e0 + j) * W + c, b);
-              acc[j] += a[0] * b[0] + a[1] * b[1] + a[2] * b[2] + a[3] * b[3];
-            }
+            acc[j] += a[0] * b[j][0] + a[1] * b[j][1] + a[2] * b[j][2] + a[3] * b[j][3];
         }
       } else {
         for (int c = threadIdx.x; c < W; c += blockDim.x) {
@@ -134,6 +140,7 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
       __syncthreads();
     }
   }
+  if (wave > 0) return;   // one wave selects: its LDS accesses are in order, no barrier is needed from here on
   const float* lrow = x ? lg : logits + (int64_t)t * EL;
   if (gate && threadIdx.x == 0) gate[t] = sigmoidf(lrow[E]);
   float sc[kMaxEPL], ch[kMaxEPL];
@@ -160,7 +167,7 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
       cs[e] = ch[i];
     }
   }
-  __syncthreads();
+  wave_sync();
   for (int g = lane; g < count; g += 64) {  // sum of the group's two largest choice scores, or the largest
     float a = -INFINITY, b = -INFINITY;
     for (int j = 0; j < per; ++j) {
@@ -170,14 +177,14 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
     }
     gs[g] = (per > 1 && rating == kRateTop2) ? a + b : a;
   }
-  __syncthreads();
+  wave_sync();
   for (int g = lane; g < count; g += 64) {  // rank among the groups (ties: the lower index first)
     int rank = 0;
     const float v = gs[g];
     for (int o = 0; o < count; ++o) rank += (gs[o] > v || (gs[o] == v && o < g)) ? 1 : 0;
     kept[g] = rank < keep ? 1 : 0;
   }
-  __syncthreads();
+  wave_sync();
 #pragma unroll
   for (int i = 0; i < kMaxEPL; ++i) {
     const int e = lane + 64 * i;
@@ -609,12 +616,16 @@ int grouped_router(const float* logits, const float* corr, int T_, int E, int co
   const int nth = x ? std::min(1024, std::max(64, ((W & 3) ? W + 63 : W / 4 + 63) / 64 * 64)) : 64;
   const int EL = E + (gate ? 1 : 0);
   const size_t lds = (E + EL + 2 * count + 16 * 16) * sizeof(float);
-  if (x && EL > 8 && EL <= 16)
-    grouped_router_kernel<16><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score,
-                                                    rating, gate);
-  else
-    grouped_router_kernel<8><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score,
-                                                   rating, gate);
+#define XGM_GR(SW)                                                                                                       \
+  grouped_router_kernel<SW><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score, rating, gate);
+  if (x && EL > 12 && EL <= 16) {
+    XGM_GR(16)
+  } else if (x && EL > 8 && EL <= 12) {
+    XGM_GR(12)
+  } else {
+    XGM_GR(8)
+  }
+#undef XGM_GR
   return 0;
 }
 

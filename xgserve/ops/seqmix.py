@@ -785,8 +785,8 @@ def glu_act(x: torch.Tensor, kind: int, limit: float = 0.0, alpha: float = 1.702
 
 
 ROUTER_FUSED_MAX_ROWS = 256     # steps of up to this many rows form the router logits inside the router kernel ...
-ROUTER_FUSED_MAX_LOGITS = 16    # ... while one sweep over the row forms them all (measured on 1 - 256 rows: 10 against 12 us
-                                # at 9 x 2048, 13 against 15 us at 9 x 4096; 13 - 18 against 12 - 15 us for 17 logits)
+ROUTER_FUSED_MAX_LOGITS = 24    # ... while one or two sweeps over the row form them all (measured on 64 rows: 8 against 12 us
+                                # for 9 x 2048, 10 against 15 us for 9 x 4096, 11 against 12 us for 17, 15 against 12 for 33)
 
 
 SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1   # grouped_router(score=...)
