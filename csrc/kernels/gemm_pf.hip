@@ -517,7 +517,7 @@ int gemm_pf_grouped(const uint16_t* x, const int32_t* rows, const int32_t* offs,
     return 1;
   if (mode == PF_PARTIAL) {
     if (part == nullptr) return 1;
-  } else if (mode == PF_BF16 || mode == PF_SILU || (mode == PF_GLU && (kind == kGluGeluTanh || kind == kGluClamped))) {
+  } else if (mode == PF_BF16 || mode == PF_SILU || (mode == PF_GLU && (kind == kGluGeluTanh || kind == kGluClamped || kind == kGluSilu))) {
     if (out == nullptr || S != 1) return 1;
   } else {
     return 1;

@@ -8,6 +8,8 @@
 //   gated_linear_scan  per head, state S [dk x dv] fp32 per (slot, head):
 //                        S_t = diag(f_t) S_(t-1) + k_t v_t^T        (k_t = 1 - f_t when k == nullptr)
 //                        o_t = S_t^T q_t
+//                      with `decay` f_t is one constant per head; with `bonus` (u, per key channel) the output reads the
+//                      state before the update, o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t;
 //                      q / f / k are fp32 tensors, or (raw form) q and f are taken straight from the fused
 //                      projection row and pass silu / the lower-bounded sigmoid while they are staged
 //
@@ -64,14 +66,17 @@ __global__ void decay_gates_kernel(const T* __restrict__ proj, int64_t ld, int o
 // through silu / the lower-bounded sigmoid while they are staged (no pass of their own, half the bytes), and the
 // write strength is 1 - f. Otherwise q, f (and k, or 1 - f when k == nullptr) are fp32 tensors [T, H dk].
 constexpr int kScanChunk = 256;
+constexpr int kScanPlain = 0, kScanRaw = 1, kScanBonus = 2;
 
-template <typename T, int NI, int TT, int NW, bool RAW, int COLS>
+template <typename T, int NI, int TT, int NW, int MODE, int COLS>
 __global__ __launch_bounds__(64 * NW) void gated_linear_scan_kernel(
     const float* __restrict__ q, const float* __restrict__ f, const float* __restrict__ k, const T* __restrict__ raw,
     int64_t ld_raw, int off_q, int off_f, const float* __restrict__ f_bias, const float* __restrict__ lower,
     const T* __restrict__ v, int64_t ld_v, float* __restrict__ state, const int32_t* __restrict__ qsl,
     const int32_t* __restrict__ seq_lens, const int32_t* __restrict__ slots, float* __restrict__ o, int H, int dk,
-    int dv, int pass, int nc, float* __restrict__ chA, float* __restrict__ chB, float* __restrict__ s_in) {
+    int dv, int pass, int nc, float* __restrict__ chA, float* __restrict__ chB, float* __restrict__ s_in,
+    const float* __restrict__ decay, const float* __restrict__ bonus) {
+  constexpr bool RAW = MODE == kScanRaw, BONUS = MODE == kScanBonus;
   constexpr int HALVES = 64 / COLS;          // row groups per wave
   constexpr int NB = NW * HALVES * NI;       // padded state rows
   constexpr int NTH = 64 * NW;
@@ -93,7 +98,11 @@ __global__ __launch_bounds__(64 * NW) void gated_linear_scan_kernel(
   const bool pok = p < dv;
   const int nqk = H * dk, nv = H * dv;
   float* Sg = state + (((int64_t)slot * H + h) * dk) * dv;
-  float S[NI], Ap[NI];
+  float S[NI], Ap[NI], un[BONUS ? NI : 1];
+  if constexpr (BONUS) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) un[i] = rg * NI + i < dk ? bonus[h * dk + rg * NI + i] : 0.f;
+  }
   const int64_t cs0 = pass ? q0 / kScanChunk + s : 0;   // the sequence's first chunk slot
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
@@ -129,7 +138,7 @@ __global__ __launch_bounds__(64 * NW) void gated_linear_scan_kernel(
             if (RAW) {
               val = ldf(raw + tok * ld_raw + (blk == 0 ? off_f : off_q) + h * dk + cc);
             } else if (blk == 0) {
-              val = f[tok * nqk + h * dk + cc];
+              val = decay ? decay[h] : f[tok * nqk + h * dk + cc];
             } else if (blk == 1) {
               val = q[tok * nqk + h * dk + cc];
             } else {
@@ -181,8 +190,14 @@ __global__ __launch_bounds__(64 * NW) void gated_linear_scan_kernel(
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
         // k = 1 - f:  f S + (1 - f) v = v + f (S - v), one operation less per element
-        S[i] = RAW ? fmaf(fr[i], S[i] - vv, vv) : fmaf(fr[i], S[i], kr[i] * vv);
-        acc = fmaf(S[i], qr[i], acc);
+        if constexpr (BONUS) {
+          const float kv = kr[i] * vv;
+          acc = fmaf(fmaf(un[i], kv, S[i]), qr[i], acc);
+          S[i] = fmaf(fr[i], S[i], kv);
+        } else {
+          S[i] = RAW ? fmaf(fr[i], S[i] - vv, vv) : fmaf(fr[i], S[i], kr[i] * vv);
+          acc = fmaf(S[i], qr[i], acc);
+        }
       }
       if (pass == 1) {   // the chunk's decay product; no outputs in this pass
 #pragma unroll
@@ -255,9 +270,11 @@ int64_t gated_linear_scan_scratch_floats(int T_, int ns, int H, int dk, int dv) 
 int gated_linear_scan(const float* q, const float* f, const float* k, const void* raw, int64_t ld_raw, int off_q, int off_f,
                       const float* f_bias, const float* lower, const void* v, bool v_f32, int64_t ld_v, float* state,
                       const int32_t* qsl, const int32_t* seq_lens, const int32_t* slots, float* o, int ns, int H, int dk,
-                      int dv, int cols_hint, float* scratch, int max_q, int T_, hipStream_t st) {
+                      int dv, int cols_hint, float* scratch, int max_q, int T_, const float* decay, const float* bonus,
+                      hipStream_t st) {
   if (ns <= 0) return 0;
-  if (H <= 0 || dk < 1 || dk > 256 || dv < 1 || (raw ? !lower : (!q || !f))) return -1;
+  if (H <= 0 || dk < 1 || dk > 256 || dv < 1 || (raw ? (!lower || decay || bonus) : (!q || (!f && !decay)))) return -1;
+  if ((decay || bonus) && !k) return -1;
   // long portions (scratch given): chunks of kScanChunk tokens over the whole grid, in two launches
   const bool chunked = scratch && max_q > kScanChunk;
   const int nc = chunked ? (max_q + kScanChunk - 1) / kScanChunk : 1;
@@ -270,28 +287,30 @@ int gated_linear_scan(const float* q, const float* f, const float* k, const void
   const bool narrow = cols_hint == 32 || (cols_hint != 64 && dv <= 32);
   const int cols = narrow ? 32 : 64;
   dim3 grid(ns * nc, H, (dv + cols - 1) / cols);
-#define XGM_GL4(NI, TT, NW, RAW, COLS, PASS)                                                                           \
-  gated_linear_scan_kernel<T, NI, TT, NW, RAW, COLS><<<grid, 64 * NW, 0, st>>>(                                         \
+#define XGM_GL4(NI, TT, NW, MODE, COLS, PASS)                                                                          \
+  gated_linear_scan_kernel<T, NI, TT, NW, MODE, COLS><<<grid, 64 * NW, 0, st>>>(                                        \
       q, f, k, (const T*)raw, ld_raw, off_q, off_f, f_bias, lower, (const T*)v, ld_v, state, qsl, seq_lens, slots, o, H, \
-      dk, dv, PASS, nc, chA, chB, s_in);
-#define XGM_GL3(NI, TT, NW, RAW, COLS)                                               \
+      dk, dv, PASS, nc, chA, chB, s_in, decay, bonus);
+#define XGM_GL3(NI, TT, NW, MODE, COLS)                                              \
   XGM_DISPATCH_T(v_f32, if (chunked) {                                               \
-    XGM_GL4(NI, TT, NW, RAW, COLS, 1)                                                \
-    XGM_GL4(NI, TT, NW, RAW, COLS, 2)                                                \
-  } else { XGM_GL4(NI, TT, NW, RAW, COLS, 0) })
+    XGM_GL4(NI, TT, NW, MODE, COLS, 1)                                               \
+    XGM_GL4(NI, TT, NW, MODE, COLS, 2)                                               \
+  } else { XGM_GL4(NI, TT, NW, MODE, COLS, 0) })
   // NI rows per lane: the narrow form covers twice the rows per wave, so it takes half of them per lane
-#define XGM_GL2(NI, TT, NW, RAW)          \
+#define XGM_GL2(NI, TT, NW, MODE)         \
   if (narrow) {                           \
-    XGM_GL3((NI / 2), TT, NW, RAW, 32)    \
+    XGM_GL3((NI / 2), TT, NW, MODE, 32)   \
   } else {                                \
-    XGM_GL3(NI, TT, NW, RAW, 64)          \
+    XGM_GL3(NI, TT, NW, MODE, 64)         \
   }
   // tokens per staged tile: the raw form stages two row blocks instead of three and takes longer tiles
 #define XGM_GL(NI, TT, TTR, NW)           \
   if (raw) {                              \
-    XGM_GL2(NI, TTR, NW, true)            \
+    XGM_GL2(NI, TTR, NW, kScanRaw)        \
+  } else if (bonus) {                     \
+    XGM_GL2(NI, TT, NW, kScanBonus)       \
   } else {                                \
-    XGM_GL2(NI, TT, NW, false)            \
+    XGM_GL2(NI, TT, NW, kScanPlain)       \
   }                                       \
   return 0;
   if (dk <= 16) { XGM_GL(4, 16, 32, 4) }

@@ -3,6 +3,7 @@
 //   glu_act          [gate | up] rows -> act(gate) * up':
 //                      kGluGeluTanh   0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * u
 //                      kGluClamped    g' = min(g, limit), u' = clamp(u, -limit, limit):  g' sigmoid(alpha g') (u' + 1)
+//                      kGluSilu       g sigmoid(g) * u
 //   grouped_router   fp32 router logits -> scores (sigmoid, or softmax over all experts); selection score = score +
 //                    correction; the experts are split into `count` contiguous groups of equal size, a group is rated
 //                    by the sum of its two highest selection scores (kRateMax: by its highest), members of the `keep`
@@ -12,6 +13,9 @@
 //                    For steps of few rows the logits x . rw[e] (fp32 rows and router weights) are formed here
 //                    by a workgroup per token, 8, 12 or 16 logits per sweep over the row, instead of being
 //                    read; its first wave then selects.
+//                    score kScoreChosen: the logits themselves compete (plus correction), and the weights are the softmax over
+//                    the `top` chosen logits alone, times scale.
+//                    bias: added to the logits that are formed here.
 //                    gate != nullptr: a logit after the experts' ones, gate[t] = sigmoid(it), takes no part in the
 //                    routing (the gate of an expert that runs for every token).
 //   moe_align        (token, choice) pairs sorted by expert into tiles of `tm` rows (padded with -1); offs: the experts'
@@ -82,7 +86,7 @@ __device__ __forceinline__ void wave_sync() {
 #endif
 }
 
-constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kRateTop2 = 0, kRateMax = 1;
+constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kScoreChosen = 2, kRateTop2 = 0, kRateMax = 1;
 
 // kRouterSweep: logits per sweep over the row when they are formed here
 template <int kRouterSweep>
@@ -90,7 +94,8 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
                                                              int E, int count, int keep, int top, float scale,
                                                              int32_t* __restrict__ ids, float* __restrict__ wts,
                                                              const float* __restrict__ x, const float* __restrict__ rw,
-                                                             int W, int score, int rating, float* __restrict__ gate) {
+                                                             int W, int score, int rating, float* __restrict__ gate,
+                                                             const float* __restrict__ bias) {
   extern __shared__ float sm[];
   float* cs = sm;              // [E] choice scores
   float* gs = sm + E;          // [count] group scores
@@ -135,7 +140,7 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
       if (threadIdx.x < kRouterSweep && e0 + threadIdx.x < EL) {
         float v = 0.f;
         for (int w = 0; w < nw; ++w) v += part[w * kRouterSweep + threadIdx.x];
-        lg[e0 + threadIdx.x] = v;
+        lg[e0 + threadIdx.x] = v + (bias ? bias[e0 + threadIdx.x] : 0.f);
       }
       __syncthreads();
     }
@@ -162,7 +167,7 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
     const int e = lane + 64 * i;
     sc[i] = 0.f, ch[i] = -INFINITY;
     if (e < E) {
-      sc[i] = score == kScoreSoftmax ? expf(lrow[e] - mx) * inv : sigmoidf(lrow[e]);
+      sc[i] = score == kScoreChosen ? lrow[e] : score == kScoreSoftmax ? expf(lrow[e] - mx) * inv : sigmoidf(lrow[e]);
       ch[i] = sc[i] + (corr ? corr[e] : 0.f);
       cs[e] = ch[i];
     }
@@ -204,15 +209,24 @@ __global__ __launch_bounds__(1024) void grouped_router_kernel(const float* __res
       const int oe = __shfl_xor(be, o, 64);
       if (ov > bv || (ov == bv && oe < be)) bv = ov, be = oe, bs = os;
     }
-    if (be >= E) be = 0, bs = 0.f;  // fewer candidates than `top`: expert 0 with weight 0
+    if (be >= E) be = 0, bs = score == kScoreChosen ? -INFINITY : 0.f;  // fewer candidates than `top`: expert 0, weight 0
     if (lane == 0) {
       ids[(int64_t)t * top + j] = be;
-      wts[(int64_t)t * top + j] = bs * scale;
+      if (score == kScoreChosen) cs[j] = bs;   // (the choice scores in LDS have been read)
+      else wts[(int64_t)t * top + j] = bs * scale;
     }
 #pragma unroll
     for (int i = 0; i < kMaxEPL; ++i)
       if (lane + 64 * i == be) ch[i] = -INFINITY;
   }
+  if (score != kScoreChosen) return;
+  wave_sync();
+  float cm = -INFINITY, sum = 0.f;
+  for (int j = lane; j < top; j += 64) cm = fmaxf(cm, cs[j]);
+  cm = wave_max(cm);
+  for (int j = lane; j < top; j += 64) sum += expf(cs[j] - cm);
+  sum = wave_sum(sum);
+  for (int j = lane; j < top; j += 64) wts[(int64_t)t * top + j] = expf(cs[j] - cm) / sum * scale;
 }
 
 // ------------------------------------------------------------------ pairs -> expert tiles (one workgroup)
@@ -606,18 +620,18 @@ void glu_act(const void* in, bool f32, int64_t ld, void* out, int T_, int F, int
 
 int grouped_router(const float* logits, const float* corr, int T_, int E, int count, int keep, int top, float scale,
                    int32_t* ids, float* wts, const float* x, const float* rw, int W, int score, int rating, float* gate,
-                   hipStream_t st) {
+                   const float* bias, hipStream_t st) {
   if (T_ <= 0) return 0;
   if (E < 1 || E > 64 * kMaxEPL || count < 1 || E % count != 0 || keep < 1 || keep > count || top < 1 ||
-      top > keep * (E / count) || score < 0 || score > 1 || rating < 0 || rating > 1)
+      top > keep * (E / count) || score < 0 || score > 2 || rating < 0 || rating > 1)
     return -1;
-  if ((x != nullptr) != (rw != nullptr) || (x && W < 1) || (!x && !logits)) return -2;
+  if ((x != nullptr) != (rw != nullptr) || (x && W < 1) || (!x && (!logits || bias))) return -2;
   // logits formed here: one pass over the row (every weight row's load in flight at once)
   const int nth = x ? std::min(1024, std::max(64, ((W & 3) ? W + 63 : W / 4 + 63) / 64 * 64)) : 64;
   const int EL = E + (gate ? 1 : 0);
   const size_t lds = (E + EL + 2 * count + 16 * 16) * sizeof(float);
 #define XGM_GR(SW)                                                                                                       \
-  grouped_router_kernel<SW><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score, rating, gate);
+  grouped_router_kernel<SW><<<T_, nth, lds, st>>>(logits, corr, E, count, keep, top, scale, ids, wts, x, rw, W, score, rating, gate, bias);
   if (x && EL > 12 && EL <= 16) {
     XGM_GR(16)
   } else if (x && EL > 8 && EL <= 12) {
@@ -643,7 +657,7 @@ int grouped_gemm(const void* A, bool f32, int64_t lda, const void* Wt, const int
                  const float* row_scale, bool mfma, hipStream_t st) {
   if (cap <= 0) return 0;
   if ((tm != 16 && tm != 32 && tm != 64 && tm != 128) || cap % tm != 0 || Nout < 1 || K < 1 || mode < kGemmRows || mode > kGemmAct ||
-      (mode == kGemmGated && kind != kGluGeluTanh && kind != kGluClamped) || (mode == kGemmAct && kind != kActRelu2) ||
+      (mode == kGemmGated && kind != kGluGeluTanh && kind != kGluClamped && kind != xgk::kGluSilu) || (mode == kGemmAct && kind != kActRelu2) ||
       (row_scale && mode != kGemmAct))
     return -1;
   if (!f32 && mfma && K % 32 == 0 && Nout % 16 == 0 && lda % 8 == 0 && (uintptr_t)A % 16 == 0 && (uintptr_t)Wt % 16 == 0) {

@@ -45,7 +45,7 @@ void lower_bound_gates(const void*, bool, int64_t, int, int, int, const float*, 
                        hipStream_t);
 int gated_linear_scan(const float*, const float*, const float*, const void*, int64_t, int, int, const float*, const float*,
                       const void*, bool, int64_t, float*, const int32_t*, const int32_t*, const int32_t*, float*, int, int,
-                      int, int, int, float*, int, int, hipStream_t);
+                      int, int, int, float*, int, int, const float*, const float*, hipStream_t);
 int64_t gated_linear_scan_scratch_floats(int, int, int, int, int);
 int ssm_scan(const void*, bool, int64_t, const void*, int64_t, const float*, const float*, const float*, float*,
              const int32_t*, const int32_t*, const int32_t*, float*, int, int, int, int, int, hipStream_t);
@@ -53,7 +53,7 @@ void gated_group_norm(const float*, const void*, bool, int64_t, const float*, in
                       hipStream_t);
 void glu_act(const void*, bool, int64_t, void*, int, int, int, float, float, hipStream_t);
 int grouped_router(const float*, const float*, int, int, int, int, int, float, int32_t*, float*, const float*, const float*,
-                   int, int, int, float*, hipStream_t);
+                   int, int, int, float*, const float*, hipStream_t);
 int hyper_residual(const float*, bool, float*, int, const void*, int64_t, bool, const float*, const float*, const int32_t*,
                    const float*, int, const float*, const float*, const float*, const float*, float, float*, void*, bool,
                    int, int, hipStream_t);
@@ -64,6 +64,18 @@ int grouped_gemm(const void*, bool, int64_t, const void*, const int32_t*, const 
 int mingru_scan(const void*, bool, int64_t, int, int, int, int, const float*, const float*, float*, const int32_t*,
                 const int32_t*, const int32_t*, void*, bool, int, int, float*, int, hipStream_t);
 int64_t mingru_scratch_floats(int, int, int);
+int layer_norm_residual(float*, const void*, int64_t, float, const void*, int64_t, float, bool, const int32_t*, int,
+                        const float*, const int32_t*, const float*, int, const float*, const float*, float, void*, bool, int,
+                        int, hipStream_t);
+void rotate_qk(const void*, bool, int64_t, int, int, int, int, const float*, int, int, float, const int32_t*, float*, float*,
+               int, hipStream_t);
+void token_shift_mix(const float*, const float*, int, float*, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
+                     void*, bool, int, int, hipStream_t);
+void time_mix_gates(const void*, int64_t, const void*, int64_t, const void*, int64_t, bool, const float*, int, float*, float*,
+                    float*, int, hipStream_t);
+int recurrent_step(const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
+                   int64_t, bool, const float*, const float*, const float*, const float*, int, int, float, const float*,
+                   float, float*, const int32_t*, const int32_t*, const int32_t*, void*, int, int, int, int, hipStream_t);
 void decay_gates(const void*, bool, int64_t, int, int, int, float, const void*, int64_t, const float*, float, float*, float*,
                  float*, int, hipStream_t);
 void moe_combine(const float*, const int32_t*, const float*, int, int, int, float*, hipStream_t);
@@ -245,7 +257,8 @@ PYBIND11_MODULE(_mixers, m) {
   m.def("gated_linear_scan", [](uintptr_t q, uintptr_t f, uintptr_t k, uintptr_t raw, int64_t ld_raw, int off_q, int off_f,
                                 uintptr_t f_bias, uintptr_t lower, uintptr_t v, bool v_f32, int64_t ld_v, uintptr_t state,
                                 uintptr_t qsl, uintptr_t sl, uintptr_t slots, uintptr_t o, int ns, int H, int dk, int dv,
-                                int cols_hint, uintptr_t scratch, int max_q, int T, uintptr_t st) {
+                                int cols_hint, uintptr_t scratch, int max_q, int T, uintptr_t decay, uintptr_t bonus,
+                                uintptr_t st) {
     if (H < 1 || dv < 1 || dk < 1 || ld_v < (int64_t)H * dv ||
         (raw && (off_q < 0 || off_f < 0 || ld_raw < off_q + (int64_t)H * dk || ld_raw < off_f + (int64_t)H * dk)))
       throw std::invalid_argument("gated_linear_scan: inconsistent sizes");
@@ -253,7 +266,7 @@ PYBIND11_MODULE(_mixers, m) {
                                     off_q, off_f, P<const float>(f_bias), P<const float>(lower), P<const void>(v), v_f32,
                                     ld_v, P<float>(state), P<const int32_t>(qsl), P<const int32_t>(sl),
                                     P<const int32_t>(slots), P<float>(o), ns, H, dk, dv, cols_hint, P<float>(scratch),
-                                    max_q, T, S(st));
+                                    max_q, T, P<const float>(decay), P<const float>(bonus), S(st));
     check(rc, "gated_linear_scan");
   });
   m.def("gated_linear_scan_scratch_floats",
@@ -278,16 +291,16 @@ PYBIND11_MODULE(_mixers, m) {
   });
   m.def("glu_act", [](uintptr_t in, bool f32, int64_t ld, uintptr_t out, int T, int F, int kind, float limit, float alpha,
                       uintptr_t st) {
-    if (kind < 0 || kind > 1 || ld < 2 * (int64_t)F) throw std::invalid_argument("glu_act: inconsistent arguments");
+    if (kind < 0 || kind > 3 || kind == 2 || ld < 2 * (int64_t)F) throw std::invalid_argument("glu_act: inconsistent arguments");
     xgm::glu_act(P<const void>(in), f32, ld, P<void>(out), T, F, kind, limit, alpha, S(st));
     check(0, "glu_act");
   });
   m.def("grouped_router", [](uintptr_t logits, uintptr_t corr, int T, int E, int count, int keep, int top, float scale,
                              uintptr_t ids, uintptr_t wts, uintptr_t x, uintptr_t rw, int W, int score, int rating,
-                             uintptr_t gate, uintptr_t st) {
+                             uintptr_t gate, uintptr_t bias, uintptr_t st) {
     int rc = xgm::grouped_router(P<const float>(logits), P<const float>(corr), T, E, count, keep, top, scale,
                                  P<int32_t>(ids), P<float>(wts), P<const float>(x), P<const float>(rw), W, score, rating,
-                                 P<float>(gate), S(st));
+                                 P<float>(gate), P<const float>(bias), S(st));
     check(rc, "grouped_router");
   });
   m.def("moe_align", [](uintptr_t ids, int pairs, int E, int cap, int tm, uintptr_t rows, uintptr_t tile_expert,
@@ -341,6 +354,59 @@ PYBIND11_MODULE(_mixers, m) {
     check(0, "decay_gates");
   });
 
+  m.def("layer_norm_residual", [](uintptr_t x, uintptr_t y1, int64_t ld1, float s1, uintptr_t y2, int64_t ld2, float s2,
+                                  bool y_f32, uintptr_t ids, int V, uintptr_t y3, uintptr_t dest, uintptr_t cw, int top,
+                                  uintptr_t w, uintptr_t next_w, float eps, uintptr_t out, bool out_f32, int T, int W,
+                                  uintptr_t st) {
+    if ((y1 && ld1 < W) || (y2 && ld2 < W)) throw std::invalid_argument("layer_norm_residual: row stride below the width");
+    int rc = xgm::layer_norm_residual(P<float>(x), P<const void>(y1), ld1, s1, P<const void>(y2), ld2, s2, y_f32,
+                                      P<const int32_t>(ids), V, P<const float>(y3), P<const int32_t>(dest),
+                                      P<const float>(cw), top, P<const float>(w), P<const float>(next_w), eps, P<void>(out),
+                                      out_f32, T, W, S(st));
+    check(rc, "layer_norm_residual");
+  });
+  m.def("rotate_qk", [](uintptr_t proj, bool f32, int64_t ld, int off_q, int off_k, int H, int dk, uintptr_t rot,
+                        int rot_rows, int rot_dims, float k_scale, uintptr_t pos, uintptr_t q, uintptr_t k, int T,
+                        uintptr_t st) {
+    const int64_t n = (int64_t)H * dk;
+    if (H < 1 || dk < 1 || off_q < 0 || off_k < 0 || ld < off_q + n || ld < off_k + n || rot_dims < 0 || rot_dims % 2 ||
+        rot_dims > dk || (rot_dims && (!rot || rot_rows < 1)))
+      throw std::invalid_argument("rotate_qk: inconsistent sizes");
+    xgm::rotate_qk(P<const void>(proj), f32, ld, off_q, off_k, H, dk, P<const float>(rot), rot_rows, rot_dims, k_scale,
+                   P<const int32_t>(pos), P<float>(q), P<float>(k), T, S(st));
+    check(0, "rotate_qk");
+  });
+  m.def("token_shift_mix", [](uintptr_t x, uintptr_t mu, int n, uintptr_t state, uintptr_t qsl, uintptr_t sl,
+                              uintptr_t slots, uintptr_t token_seq, uintptr_t out, bool out_f32, int T, int W,
+                              uintptr_t st) {
+    if (n < 1 || W < 1) throw std::invalid_argument("token_shift_mix: inconsistent sizes");
+    xgm::token_shift_mix(P<const float>(x), P<const float>(mu), n, P<float>(state), P<const int32_t>(qsl),
+                         P<const int32_t>(sl), P<const int32_t>(slots), P<const int32_t>(token_seq), P<void>(out), out_f32,
+                         T, W, S(st));
+    check(0, "token_shift_mix");
+  });
+  m.def("time_mix_gates", [](uintptr_t r, int64_t ld_r, uintptr_t k, int64_t ld_k, uintptr_t z, int64_t ld_z, bool f32,
+                             uintptr_t w0, int n, uintptr_t ro, uintptr_t fo, uintptr_t ko, int T, uintptr_t st) {
+    if (n < 1 || ld_r < n || ld_k < n || ld_z < n) throw std::invalid_argument("time_mix_gates: inconsistent sizes");
+    xgm::time_mix_gates(P<const void>(r), ld_r, P<const void>(k), ld_k, P<const void>(z), ld_z, f32, P<const float>(w0), n,
+                        P<float>(ro), P<float>(fo), P<float>(ko), T, S(st));
+    check(0, "time_mix_gates");
+  });
+  m.def("recurrent_step", [](uintptr_t q, int64_t ld_q, uintptr_t k, int64_t ld_k, uintptr_t v, int64_t ld_v, uintptr_t g,
+                             int64_t ld_g, uintptr_t z, int64_t ld_z, bool f32, uintptr_t decay, uintptr_t w0,
+                             uintptr_t bonus, uintptr_t rot, int rot_rows, int rot_dims, float k_scale, uintptr_t norm_w,
+                             float eps, uintptr_t state, uintptr_t sl, uintptr_t slots, uintptr_t pos, uintptr_t out, int ns,
+                             int H, int dk, int dv, uintptr_t st) {
+    const int64_t nk = (int64_t)H * dk, nv = (int64_t)H * dv;
+    if (ld_q < nk || ld_k < nk || ld_v < nv || ld_g < nv || (z && ld_z < nk) || rot_dims < 0 || (rot_dims && rot_rows < 1))
+      throw std::invalid_argument("recurrent_step: inconsistent sizes");
+    int rc = xgm::recurrent_step(P<const void>(q), ld_q, P<const void>(k), ld_k, P<const void>(v), ld_v, P<const void>(g),
+                                 ld_g, P<const void>(z), ld_z, f32, P<const float>(decay), P<const float>(w0),
+                                 P<const float>(bonus), P<const float>(rot), rot_rows, rot_dims, k_scale,
+                                 P<const float>(norm_w), eps, P<float>(state), P<const int32_t>(sl), P<const int32_t>(slots),
+                                 P<const int32_t>(pos), P<void>(out), ns, H, dk, dv, S(st));
+    check(rc, "recurrent_step");
+  });
   m.def("canon_conv", [](uintptr_t x, uintptr_t w, uintptr_t state, uintptr_t qsl, uintptr_t sl, uintptr_t slots,
                          uintptr_t out, bool out_f32, int ns, int max_q, int W, int taps, uintptr_t st) {
     if (taps < 1 || taps > 8) throw std::invalid_argument("canon_conv: taps must be in [1, 8]");

@@ -8,7 +8,7 @@
 //                     x / B / C are columns of one activation row [x (H P) | B (G N) | C (G N)] (already
 //                     through their short convolution and activation), dt_raw a column block of another.
 //   gated_group_norm  v = y * silu(z) (v = y without z);  each of `ng` equal parts of v divided by its own root
-//                     mean square, times w (gated first, normed second); w repeats with period wn. With
+//                     mean square, times w (gated first, normed second); w (nullptr = 1) repeats with period wn. With
 //                     `gate_after` the norm is taken of y itself and silu(z) multiplies the normed, weighted result.
 //
 // One workgroup = (sequence, head, 64 state columns), NW waves: lane p owns column p, wave w owns rows
@@ -150,7 +150,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
   for (int c = threadIdx.x; c < gs; c += blockDim.x) {
     float v = y[(int64_t)t * inner + c0 + c];
     if (pre) v *= siluf(ldf(z + (int64_t)t * ld_z + c0 + c));
-    v = v * r * w[(c0 + c) % wn];
+    v = v * r * (w ? w[(c0 + c) % wn] : 1.f);
     if (post) v *= siluf(ldf(z + (int64_t)t * ld_z + c0 + c));
     stf(out + (int64_t)t * inner + c0 + c, v);
   }

@@ -16,7 +16,7 @@ from typing import Dict, List, Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str                      # "llama" | "mixtral" | "gpt2" | "dofivik" | "vizonex" | "loluzen" | "lotelix" | "taritar"
+    arch: str                      # "llama" | "mixtral" | "gpt2" | "dofivik" | "vizonex" | "loluzen" | "lotelix" | "taritar" | "bazurax"
     hidden_size: int
     num_layers: int
     num_heads: int
@@ -69,6 +69,8 @@ class ModelConfig:
                 from .lotelix import count_params
             elif self.arch == "taritar":
                 from .taritar import count_params
+            elif self.arch == "bazurax":
+                from .bazurax import count_params
             else:
                 from .dofivik import count_params
             return count_params(self)
@@ -97,6 +99,9 @@ class ModelConfig:
             return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes for m in att)
         if self.arch == "lotelix":
             att = [(L["mixer"].get("left") or L["mixer"]) for L in self.layer_specs if L["type"] != "mingru"]
+            return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes for m in att)
+        if self.arch == "bazurax":
+            att = [L["mixer"]["left"] for L in self.layer_specs if L["type"] == "parallel"]
             return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes for m in att)
         if self.arch in ("vizonex", "taritar"):   # (a layer that reads another layer's keys and values caches nothing)
             return sum((m["dim"] + m["vdim"]) * m["kv_heads"] * dtype_bytes
@@ -487,6 +492,81 @@ def _taritar_tiny_layers():
 
 register(taritar_config("taritar-tiny", 128, 512, _taritar_tiny_layers(), streams=3, embed_scale=2.0, logit_softcap=25.0,
                         max_position=1024))
+def bazurax_config(name: str, width: int, vocab: int, layers: List[dict], eps: float = 1e-6,
+                   max_position: int = 131072) -> ModelConfig:
+    """A Bazurax model: layers x <- x + L(mixer(x)), x <- x + L(ff(x)) with a layer norm L on each sublayer's output and on
+    the embedding rows; the output matrix is the embedding table. Mixers: "retention" (linear attention with a constant decay
+    per head on rotated queries and keys) and "parallel" (a weighted sum of sliding-window attention with whole-projection
+    q / k norms and one output gate per head, and a time-mixing recurrence with token shift, a data-dependent decay per key
+    channel and a bonus for the current token). Feed-forward: a silu-gated one, dense or as routed experts whose weights are
+    the softmax over the chosen router logits, or none."""
+    def need(d, keys, where):
+        for k in keys:
+            if k not in d:
+                raise ValueError(f"{where}: missing {k!r}")
+    if not layers:
+        raise ValueError("a model needs at least one layer")
+    if width > 16000:
+        raise ValueError("widths above 16000 are not supported")
+    for i, L in enumerate(layers):
+        m, w = L.get("mixer") or {}, f"layer {i}"
+        if L.get("type") == "retention":
+            need(m, ("heads", "dim", "vdim", "decay"), w)
+            if m["heads"] < 1 or len(m["decay"]) != m["heads"]:
+                raise ValueError(f"{w}: needs one decay per head")
+            if not 1 <= m["dim"] <= 256 or not 1 <= m["vdim"] <= 8192:
+                raise ValueError(f"{w}: recurrent head sizes above 256 (value sizes above 8192) are not supported")
+            rot = m.get("rot")
+            if rot is not None:
+                need(rot, ("base", "dims"), w)
+                if rot["dims"] % 2 or not 0 <= rot["dims"] <= m["dim"]:
+                    raise ValueError(f"{w}: rot.dims must be even and at most dim")
+        elif L.get("type") == "parallel":
+            need(m, ("left", "right", "left_scale", "right_scale"), w)
+            a, r = m["left"], m["right"]
+            need(a, ("heads", "kv_heads", "dim", "vdim", "scale"), w + " left")
+            if a["heads"] < 1 or a["kv_heads"] < 1 or a["heads"] % a["kv_heads"]:
+                raise ValueError(f"{w} left: heads must be a positive multiple of kv_heads")
+            if a.get("mask") is not None and int(a["mask"]["size"]) < 1:
+                raise ValueError(f"{w} left: mask.size must be positive")
+            need(r, ("heads", "dim"), w + " right")
+            if r["heads"] < 1 or not 1 <= r["dim"] <= 256:
+                raise ValueError(f"{w} right: recurrent head sizes above 256 are not supported")
+        else:
+            raise ValueError(f"{w}: unknown mixer type {L.get('type')!r}")
+        mlp = L.get("mlp")
+        if mlp is None:
+            continue
+        if mlp.get("kind") == "dense":
+            need(mlp, ("ff",), w)
+        elif mlp.get("kind") == "moe":
+            need(mlp, ("expert", "router"), w)
+            need(mlp["expert"], ("ff",), w)
+            need(mlp["router"], ("experts", "top"), w)
+            if not 1 <= mlp["router"]["top"] <= mlp["router"]["experts"] <= 512:
+                raise ValueError(f"{w}: needs 1 <= top <= experts <= 512")
+        else:
+            raise ValueError(f"{w}: unknown feed-forward kind {mlp.get('kind')!r}")
+    att = [L["mixer"]["left"] for L in layers if L["type"] == "parallel"]
+    ffs = [(L["mlp"]["ff"] if L["mlp"]["kind"] == "dense" else L["mlp"]["expert"]["ff"] * L["mlp"]["router"]["top"])
+           for L in layers if L.get("mlp")]
+    return ModelConfig(name, "bazurax", width, len(layers), max([m["heads"] for m in att] or [1]),
+                       max([m["kv_heads"] for m in att] or [1]), max([max(m["dim"], m["vdim"]) for m in att] or [1]),
+                       max(ffs or [0]), vocab, max_position, 0.0, None, eps, True, bos_token_id=0, eos_token_ids=[],
+                       layer_specs=layers)
+
+
+def _bazurax_tiny_layers():
+    ret = {"heads": 3, "dim": 32, "vdim": 48, "decay": [0.9, 0.98, 0.995], "rot": {"base": 10000.0, "dims": 16}}
+    par = {"left": {"heads": 4, "kv_heads": 2, "dim": 32, "vdim": 16, "scale": 0.2, "mask": {"size": 24}},
+           "right": {"heads": 2, "dim": 32, "decay_rank": 8}, "left_scale": 0.75, "right_scale": 1.5}
+    moe = {"kind": "moe", "expert": {"ff": 48}, "router": {"experts": 6, "top": 2}}
+    return [{"type": "retention", "mixer": dict(ret), "mlp": {"kind": "dense", "ff": 160}},
+            {"type": "parallel", "mixer": par, "mlp": dict(moe)},
+            {"type": "retention", "mixer": dict(ret), "mlp": None}]
+
+
+register(bazurax_config("bazurax-tiny", 128, 512, _bazurax_tiny_layers(), max_position=1024))
 register(ModelConfig("gpt2-tiny", "gpt2", 128, 2, 2, 2, 64, 512, 512, 256, 0.0, tie_embeddings=True,
                      bos_token_id=0, eos_token_ids=[0], dtype="float32"))
 
@@ -522,6 +602,9 @@ def from_hf_config(path: str, name: Optional[str] = None) -> ModelConfig:
         return taritar_config(name or "taritar", c["width"], c["vocab"], c["layers"], int(c["streams"]),
                               c["embedding"]["scale"], c["norm"]["eps"], c.get("logit_softcap"),
                               int(c.get("max_positions", 4096)))
+    if c.get("architecture") == "Bazurax":
+        return bazurax_config(name or "bazurax", c["width"], c["vocab"], c["layers"], c["norm"]["eps"],
+                              int(c.get("max_position", 131072)))
     mt = c.get("model_type", "llama")
     eos = c.get("eos_token_id", 2)
     eos = eos if isinstance(eos, list) else [eos]

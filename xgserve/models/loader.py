@@ -18,6 +18,7 @@ import torch
 
 from ..ops.linear import deinterleave_gate_up, interleave_gate_up
 from .base import kv_head_range
+from .bazurax import BazuraxForCausalLM
 from .config import ModelConfig, get_config
 from .dofivik import DofivikForCausalLM
 from .gpt2 import GPT2ForCausalLM
@@ -30,13 +31,20 @@ from .vizonex import VizonexForCausalLM
 
 def model_class(cfg: ModelConfig):
     return {"gpt2": GPT2ForCausalLM, "dofivik": DofivikForCausalLM, "vizonex": VizonexForCausalLM,
-            "loluzen": LoluzenForCausalLM, "lotelix": LotelixForCausalLM, "taritar": TaritarForCausalLM}.get(cfg.arch, LlamaForCausalLM)
+            "loluzen": LoluzenForCausalLM, "lotelix": LotelixForCausalLM, "taritar": TaritarForCausalLM,
+            "bazurax": BazuraxForCausalLM}.get(cfg.arch, LlamaForCausalLM)
 
 
 def _resolve_shapes(cfg: ModelConfig, checkpoint: str) -> None:
     """Sizes that only a tensor's shape gives (Dofivik: the rank of the decay projection; Loluzen: the taps of
     a short convolution when the configuration leaves them out; Lotelix: the rank of the decay projection;
-    Taritar: the number of learned positions)."""
+    Taritar: the number of learned positions; Bazurax: the rank of the decay projection)."""
+    if cfg.arch == "bazurax":
+        r = _Reader(checkpoint)
+        for i, spec in enumerate(cfg.layer_specs):
+            if spec["type"] == "parallel":
+                spec["mixer"]["right"]["decay_rank"] = int(r.shape(f"l{i}.mix.right.w1")[0])
+        return
     if cfg.arch == "taritar":
         cfg.max_position = int(_Reader(checkpoint).shape("pos")[0])
         return
@@ -150,6 +158,8 @@ def load_checkpoint(model, path: str) -> None:
         _load_lotelix(model, r)
     elif cfg.arch == "taritar":
         _load_taritar(model, r)
+    elif cfg.arch == "bazurax":
+        _load_bazurax(model, r)
     else:
         _load_llama(model, r)
 
@@ -505,6 +515,78 @@ def _save_taritar(model, path: str) -> None:
                    "max_positions": cfg.max_position}, f, indent=1)
 
 
+def _bazurax_tensors(m):
+    """(checkpoint name, parameter, index of a fused / stacked parameter or None) for every tensor."""
+    out = [("embed", m.embed, None), ("embed.norm", m.embed_norm, None), ("final.norm", m.final_norm, None)]
+
+    def rows(pre, p, parts):
+        at = 0
+        for name, n in parts:
+            out.append((pre + name, p, slice(at, at + n)))
+            at += n
+    for i, L in enumerate(m.layers):
+        b, x = f"l{i}.", L.mix
+        out.append((b + "norm1", L.norm1, None))
+        if L.kind == "retention":
+            rows(b + "mix.", x.in_proj, (("q", x.n), ("k", x.n), ("v", x.nv), ("g", x.nv)))
+            out.append((b + "mix.o", x.o, None))
+        else:
+            a, r = x.left, x.right
+            rows(b + "mix.left.", a.in_proj, (("q", a.nq), ("k", a.nk), ("v", a.nv), ("g", a.H)))
+            out += [(b + "mix.left.q.norm", a.q_norm, None), (b + "mix.left.k.norm", a.k_norm, None), (b + "mix.left.o", a.o, None)]
+            c = b + "mix.right."
+            out += [(c + "mu." + s, r.mu, j) for j, s in enumerate("rkvgw")]
+            out += [(c + s, r.rkvg, j) for j, s in enumerate("rkvg")]
+            out += [(c + "w1", r.w1, None), (c + "w2", r.w2, None), (c + "w0", r.w0, None), (c + "u", r.u, "heads"),
+                    (c + "norm", r.norm, None), (c + "o", r.o, None)]
+        if L.mlp is None:
+            continue
+        out.append((b + "norm2", L.norm2, None))
+        F_ = L.mlp.ff
+        if not L.moe:
+            rows(b + "mlp.", L.mlp.gate_up, (("gate", F_), ("up", F_)))
+            out.append((b + "mlp.down", L.mlp.down, None))
+            continue
+        out += [(b + "mlp.router", L.mlp.router, None), (b + "mlp.router.b", L.mlp.router_b, None)]
+        for e in range(L.mlp.E):
+            out += [(f"{b}mlp.e{e}.gate", L.mlp.w13, (e, slice(0, F_))), (f"{b}mlp.e{e}.up", L.mlp.w13, (e, slice(F_, 2 * F_))),
+                    (f"{b}mlp.e{e}.down", L.mlp.w2, e)]
+    return out
+
+
+def _load_bazurax(m, r: _Reader):
+    """Tensors `embed` (also the output matrix), `embed.norm`, `final.norm`, `l<i>.<norm1|norm2>`, `l<i>.mix.*`, `l<i>.mlp.*`
+    ([out, in] matrices). Projections that read the same input and gate / up are fused row-wise; the time-mixing shares and
+    projections, and the experts, stacked, on load."""
+    for name, p, idx in _bazurax_tensors(m):
+        src = r.get(name)
+        if idx == "heads":   # [heads, dim], kept flat
+            src, idx = src.reshape(-1), None
+        dst = p.data if idx is None else p.data[idx]
+        if tuple(dst.shape) != tuple(src.shape):
+            raise ValueError(f"shape mismatch for {name}: model {tuple(dst.shape)} vs checkpoint {tuple(src.shape)}")
+        dst.copy_(src.to(dst.dtype))
+
+
+def _save_bazurax(model, path: str) -> None:
+    from safetensors.torch import save_file
+    cfg = model.cfg
+    t, layers = {}, []
+    heads = {f"l{i}.mix.right.u": L.mix.right.H for i, L in enumerate(model.layers) if L.kind == "parallel"}
+    for name, p, idx in _bazurax_tensors(model):
+        v = p.data.view(heads[name], -1) if idx == "heads" else p.data if idx is None else p.data[idx]
+        t[name] = v.detach().to(torch.bfloat16).contiguous().cpu()
+    save_file(t, os.path.join(path, "model.safetensors"))
+    for spec in cfg.layer_specs:
+        mx = dict(spec["mixer"])
+        if spec["type"] == "parallel":   # the rank of the decay projection is given by a tensor's shape
+            mx["right"] = {k: v for k, v in mx["right"].items() if k != "decay_rank"}
+        layers.append({"type": spec["type"], "mixer": mx, "mlp": spec.get("mlp")})
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump({"architecture": "Bazurax", "width": cfg.hidden_size, "vocab": cfg.vocab_size, "layers": layers,
+                   "norm": {"eps": cfg.norm_eps}, "max_position": cfg.max_position}, f, indent=1)
+
+
 def _save_vizonex(model, path: str) -> None:
     from safetensors.torch import save_file
     cfg = model.cfg
@@ -554,6 +636,8 @@ def save_checkpoint(model, path: str) -> None:
         return _save_lotelix(model, path)
     if cfg.arch == "taritar":
         return _save_taritar(model, path)
+    if cfg.arch == "bazurax":
+        return _save_bazurax(model, path)
     t: Dict[str, torch.Tensor] = {}
     if cfg.arch == "gpt2":
         t["transformer.wte.weight"] = model.wte

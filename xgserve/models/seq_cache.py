@@ -26,7 +26,8 @@ class LayerCache:
     delta: Optional[torch.Tensor] = None    # delta rule: [slots, heads, dim, dim]
     mix_conv: Optional[torch.Tensor] = None  # a mixer's own short convolution: [slots, taps - 1, channels]
     ssm: Optional[torch.Tensor] = None      # state-space recurrence: [slots, heads, state, vdim]
-    gla: Optional[torch.Tensor] = None      # gated linear recurrence: [slots, heads, dim, vdim]
+    gla: Optional[torch.Tensor] = None      # linear recurrence (gated, retention, time mixing): [slots, heads, dim, vdim]
+    shift: Optional[torch.Tensor] = None    # token shift: [slots, width], a mixer's input at the last token
     gru: Optional[torch.Tensor] = None      # minimal gated recurrence: [slots, width]
 
 

@@ -719,14 +719,14 @@ def ssm_scan(xbc: torch.Tensor, dt_raw: torch.Tensor, dt_bias: torch.Tensor, A_l
     return y
 
 
-def gated_group_norm(y: torch.Tensor, z: Optional[torch.Tensor], w: torch.Tensor, eps: float, groups: int,
+def gated_group_norm(y: torch.Tensor, z: Optional[torch.Tensor], w: Optional[torch.Tensor], eps: float, groups: int,
                      out_dtype: torch.dtype, gate_after: bool = False) -> torch.Tensor:
     """v = y * silu(z) (v = y when z is None); each of `groups` equal parts of a row divided by its own root mean
     square; times w, which holds one weight per column or one period of a repeating pattern (e.g. a weight of one
-    head's size shared by all heads). With `gate_after` the norm is taken of y itself and silu(z) multiplies the
+    head's size shared by all heads; None: no weight). With `gate_after` the norm is taken of y itself and silu(z) multiplies the
     normed, weighted result. y fp32 [T, n]; z [T, n] (row-strided activation)."""
     T, n = y.shape
-    assert n % groups == 0 and n % w.numel() == 0
+    assert n % groups == 0 and (w is None or n % w.numel() == 0)
     if not native_device(y):
         v = y
         gate = None
@@ -736,20 +736,22 @@ def gated_group_norm(y: torch.Tensor, z: Optional[torch.Tensor], w: torch.Tensor
             if not gate_after:
                 v = y * gate
         v = v.view(T, groups, n // groups)
-        v = (v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)).reshape(T, n) * w.repeat(n // w.numel())
+        v = (v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)).reshape(T, n)
+        if w is not None:
+            v = v * w.repeat(n // w.numel())
         if gate_after and gate is not None:
             v = v * gate
         return v.to(out_dtype)
     out = torch.empty(T, n, dtype=out_dtype, device=y.device)
-    assert y.is_contiguous() and y.dtype == torch.float32 and w.dtype == torch.float32
+    assert y.is_contiguous() and y.dtype == torch.float32 and (w is None or w.dtype == torch.float32)
     assert z is None or (z.stride(1) == 1 and z.dtype == out_dtype)
-    mixers().gated_group_norm(y.data_ptr(), _p(z), is_f32(out), z.stride(0) if z is not None else 0, w.data_ptr(),
-                              w.numel(), float(eps), out.data_ptr(), T, n, groups, bool(gate_after), stream_ptr())
+    mixers().gated_group_norm(y.data_ptr(), _p(z), is_f32(out), z.stride(0) if z is not None else 0, _p(w),
+                              w.numel() if w is not None else 1, float(eps), out.data_ptr(), T, n, groups, bool(gate_after), stream_ptr())
     return out
 
 
 # ---------------------------------------------------------------------------- gated feed-forward, routed experts
-GLU_GELU_TANH, GLU_CLAMPED = 0, 1
+GLU_GELU_TANH, GLU_CLAMPED, GLU_SILU = 0, 1, 3
 ACT_RELU2 = 2   # routed_experts(kind=...): an expert without a gate, W_down relu(W_up h)^2
 # XGS_TUNE moe_mfma=0: the general grouped GEMM for bf16 too (A/B and tests)
 MOE_MFMA = tune.get_bool("moe_mfma", True)
@@ -764,6 +766,8 @@ MOE_TILE32_MIN = tune.get_int("moe_tile32_min", MOE_TILE32_MIN)
 def _glu_ref(g, u, kind, limit, alpha):
     if kind == GLU_GELU_TANH:
         return 0.5 * g * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (g + 0.044715 * g ** 3))) * u
+    if kind == GLU_SILU:
+        return g * torch.sigmoid(g) * u
     g = g.clamp(max=limit)
     u = u.clamp(-limit, limit)
     return g * torch.sigmoid(alpha * g) * (u + 1.0)
@@ -771,7 +775,7 @@ def _glu_ref(g, u, kind, limit, alpha):
 
 def glu_act(x: torch.Tensor, kind: int, limit: float = 0.0, alpha: float = 1.702) -> torch.Tensor:
     """Rows [gate (F) | up (F)] -> [F]: GLU_GELU_TANH: gelu_tanh(gate) * up; GLU_CLAMPED: with g = min(gate, limit),
-    u = clamp(up, -limit, limit): g * sigmoid(alpha g) * (u + 1)."""
+    u = clamp(up, -limit, limit): g * sigmoid(alpha g) * (u + 1); GLU_SILU: silu(gate) * up."""
     T, F2 = x.shape
     F_ = F2 // 2
     if not native_device(x):
@@ -789,17 +793,19 @@ ROUTER_FUSED_MAX_LOGITS = 24    # ... while one or two sweeps over the row form 
                                 # for 9 x 2048, 10 against 15 us for 9 x 4096, 11 against 12 us for 17, 15 against 12 for 33)
 
 
-SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1   # grouped_router(score=...)
+SCORE_SIGMOID, SCORE_SOFTMAX, SCORE_CHOSEN = 0, 1, 2   # grouped_router(score=...)
 RATE_TOP2, RATE_MAX = 0, 1            # grouped_router(rating=...): how a group of experts is rated
 
 
 def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Tensor], count: int, keep: int, top: int,
                    scale: float, rows: Optional[torch.Tensor] = None, router_w: Optional[torch.Tensor] = None,
-                   score: int = SCORE_SIGMOID, rating: int = RATE_TOP2, extra_gate: bool = False, want_gate: bool = False):
+                   score: int = SCORE_SIGMOID, rating: int = RATE_TOP2, extra_gate: bool = False, want_gate: bool = False,
+                   bias: Optional[torch.Tensor] = None):
     """fp32 router logits [T, E] -> (expert ids int32 [T, top], weights fp32 [T, top]). With `rows` (fp32 [T, W]) and
     `router_w` (fp32 [E, W]) in place of `logits` the logits are rows . router_w[e] in fp32: inside the router kernel
     for steps of few rows on the GPU (a launch less; the library product wins on long steps), else a matrix product. Scores are
-    sigmoid(logits), or with SCORE_SOFTMAX their softmax over all experts. Selection uses score + correction: the experts form `count` contiguous groups of equal
+    sigmoid(logits), with SCORE_SOFTMAX their softmax over all experts, or with SCORE_CHOSEN the logits themselves, whose
+    softmax over the chosen experts alone gives the weights. `bias` (fp32 [logits]) is added to logits formed here. Selection uses score + correction: the experts form `count` contiguous groups of equal
     size, a group is rated by the sum of its two highest selection scores (RATE_MAX: by its highest), and only members of
     the `keep` highest-rated groups are eligible (everything else is excluded outright, selection score -inf). The
     returned weights are score * scale: the correction does not enter them and they are not normalised.
@@ -811,13 +817,15 @@ def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Te
         fused = native_device(rows) and rows.shape[0] <= ROUTER_FUSED_MAX_ROWS and rows.is_contiguous() \
             and router_w.is_contiguous() and router_w.shape[0] <= ROUTER_FUSED_MAX_LOGITS
         if not fused:
-            logits = torch.nn.functional.linear(rows, router_w)
+            logits = torch.nn.functional.linear(rows, router_w, bias)
+    else:
+        assert bias is None
     T, E = (rows.shape[0], router_w.shape[0]) if fused else logits.shape
     E -= int(extra_gate)
     if not fused and not native_device(logits):
         gate = torch.sigmoid(logits[:, E].float()) if extra_gate else None
         z = logits[:, :E].float()
-        s = torch.softmax(z, -1) if score == SCORE_SOFTMAX else torch.sigmoid(z)
+        s = z if score == SCORE_CHOSEN else torch.softmax(z, -1) if score == SCORE_SOFTMAX else torch.sigmoid(z)
         c = s + (correction if correction is not None else 0.0)
         per = E // count
         gsc = c.view(T, count, per).topk(1 if rating == RATE_MAX else min(2, per), -1).values.sum(-1)
@@ -825,7 +833,8 @@ def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Te
         kept.scatter_(1, gsc.topk(keep, -1).indices, True)
         c = c.masked_fill(~kept.repeat_interleave(per, 1), float("-inf"))
         ids = c.topk(top, -1).indices
-        ids, wts = ids.to(torch.int32), s.gather(1, ids) * scale
+        wts = s.gather(1, ids)
+        ids, wts = ids.to(torch.int32), (torch.softmax(wts, -1) if score == SCORE_CHOSEN else wts) * scale
         return (ids, wts, gate) if want_gate else (ids, wts)
     assert fused or (logits.dtype == torch.float32 and logits.is_contiguous())
     dev = rows.device if fused else logits.device
@@ -835,7 +844,7 @@ def grouped_router(logits: Optional[torch.Tensor], correction: Optional[torch.Te
     mixers().grouped_router(0 if fused else logits.data_ptr(), _p(correction), T, E, int(count), int(keep), int(top),
                             float(scale), ids.data_ptr(), wts.data_ptr(), rows.data_ptr() if fused else 0,
                             router_w.data_ptr() if fused else 0, rows.shape[1] if fused else 0, int(score), int(rating),
-                            _p(gate), stream_ptr())
+                            _p(gate), _p(bias) if fused else 0, stream_ptr())
     return (ids, wts, gate) if want_gate else (ids, wts)
 
 
@@ -863,7 +872,7 @@ def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: to
     Returns fp32 [T, W] (a sum in a fixed order per row), or with combine=False the rows as `RoutedRows`."""
     T, K = h.shape
     E = w13.shape[0]
-    gated = kind in (GLU_GELU_TANH, GLU_CLAMPED)
+    gated = kind in (GLU_GELU_TANH, GLU_CLAMPED, GLU_SILU)
     F_ = w13.shape[1] // 2 if gated else w13.shape[1]
     W, top = w2.shape[1], ids.shape[1]
     if not native_device(h):
@@ -1130,24 +1139,30 @@ def lower_bound_gates(proj: torch.Tensor, off_q: int, off_f: int, n: int, f_bias
     return qf[0], qf[1]
 
 
-def gated_linear_scan(q: torch.Tensor, f: torch.Tensor, k: Optional[torch.Tensor], v: torch.Tensor, state: torch.Tensor,
-                      H: int, dk: int, dv: int, sm: SeqMeta) -> torch.Tensor:
+def gated_linear_scan(q: torch.Tensor, f: Optional[torch.Tensor], k: Optional[torch.Tensor], v: torch.Tensor,
+                      state: torch.Tensor, H: int, dk: int, dv: int, sm: SeqMeta, decay: Optional[torch.Tensor] = None,
+                      bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per head a [dk x dv] fp32 state with one decay per row:  S <- diag(f) S + k v^T,  o = S^T q;  k = 1 - f when
-    `k` is None (write strength = complement of the forget gate). q, f, k fp32 [T, H dk]; v [T, H dv] (row-strided
-    activation). state fp32 [slots, H, dk, dv] is carried and updated. Returns o fp32 [T, H dv]."""
+    `k` is None (write strength = complement of the forget gate). With `decay` (fp32 [H]) f is that constant per head
+    (f None); with `bonus` (u, fp32 [H dk]) the output reads the state before the update, o = (S + diag(u) k v^T)^T q
+    (both need k). q, f, k fp32 [T, H dk]; v [T, H dv] (row-strided activation). state fp32 [slots, H, dk, dv] is carried and updated. Returns o fp32 [T, H dv]."""
     T = q.shape[0]
     o = torch.empty(T, H * dv, dtype=torch.float32, device=q.device)
     if native_device(q):
-        assert q.dtype == f.dtype == torch.float32 and q.is_contiguous() and f.is_contiguous() and v.stride(1) == 1
+        assert q.dtype == torch.float32 and q.is_contiguous() and v.stride(1) == 1
+        assert (f is None) == (decay is not None) and (f is None or (f.dtype == torch.float32 and f.is_contiguous()))
+        assert decay is None or (decay.dtype == torch.float32 and decay.numel() == H)
+        assert bonus is None or (bonus.dtype == torch.float32 and bonus.is_contiguous() and bonus.numel() == H * dk)
         assert k is None or (k.dtype == torch.float32 and k.is_contiguous())
         assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, dk, dv)
         scratch = _scan_scratch(T, sm, H, dk, dv, q.device)
-        mixers().gated_linear_scan(q.data_ptr(), f.data_ptr(), _p(k), 0, 0, 0, 0, 0, 0, v.data_ptr(), is_f32(v),
+        mixers().gated_linear_scan(q.data_ptr(), _p(f), _p(k), 0, 0, 0, 0, 0, 0, v.data_ptr(), is_f32(v),
                                    v.stride(0), state.data_ptr(), _i32(sm.qsl).data_ptr(), _i32(sm.seq_lens).data_ptr(),
                                    _i32(sm.slots).data_ptr(), o.data_ptr(), sm.num_seqs, H, dk, dv, SCAN_COLS,
-                                   _p(scratch), sm.max_q, T, stream_ptr())
+                                   _p(scratch), sm.max_q, T, _p(decay), _p(bonus), stream_ptr())
         return o
-    qh, fh = q.view(T, H, dk), f.view(T, H, dk)
+    qh = q.view(T, H, dk)
+    fh = f.view(T, H, dk) if decay is None else decay[None, :, None].expand(T, H, dk)
     kh = (1.0 - fh) if k is None else k.view(T, H, dk)
     vh = v.float().reshape(T, H, dv)
     qsl, sl, slots = sm.qsl.tolist(), sm.seq_lens.tolist(), sm.slots.tolist()
@@ -1157,8 +1172,12 @@ def gated_linear_scan(q: torch.Tensor, f: torch.Tensor, k: Optional[torch.Tensor
             continue
         S = state[slots[s]].clone() if sl[s] - (hi - lo) > 0 else torch.zeros(H, dk, dv)
         for t in range(lo, hi):
-            S = fh[t][:, :, None] * S + kh[t][:, :, None] * vh[t][:, None, :]
-            o[t] = torch.einsum("hkd,hk->hd", S, qh[t]).reshape(H * dv)
+            kv = kh[t][:, :, None] * vh[t][:, None, :]
+            if bonus is not None:
+                o[t] = torch.einsum("hkd,hk->hd", S + bonus.view(H, dk, 1) * kv, qh[t]).reshape(H * dv)
+            S = fh[t][:, :, None] * S + kv
+            if bonus is None:
+                o[t] = torch.einsum("hkd,hk->hd", S, qh[t]).reshape(H * dv)
         state[slots[s]] = S
     return o
 
@@ -1179,7 +1198,7 @@ def lower_bound_recurrence(proj: torch.Tensor, off_q: int, off_f: int, off_v: in
     mixers().gated_linear_scan(0, 0, 0, proj.data_ptr(), proj.stride(0), off_q, off_f, _p(f_bias), lower.data_ptr(),
                                v.data_ptr(), is_f32(proj), proj.stride(0), state.data_ptr(), _i32(sm.qsl).data_ptr(),
                                _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(), o.data_ptr(), sm.num_seqs, H, dk,
-                               dv, SCAN_COLS, _p(scratch), sm.max_q, proj.shape[0], stream_ptr())
+                               dv, SCAN_COLS, _p(scratch), sm.max_q, proj.shape[0], 0, 0, stream_ptr())
     return o
 
 
@@ -1258,3 +1277,164 @@ def decay_gates(proj: torch.Tensor, off_q: int, off_k: int, n: int, q_scale: flo
                          z.stride(0), _p(z_bias), float(1.0 / tau), out[0].data_ptr(), out[1].data_ptr(),
                          out[2].data_ptr(), T, stream_ptr())
     return out[0], out[1], out[2]
+
+
+# ---------------------------------------------------------------------------- layer norm on a sublayer's output
+def layer_norm_residual(x: Optional[torch.Tensor], y, w: torch.Tensor, eps: float, out_dtype: torch.dtype,
+                        y2: Optional[torch.Tensor] = None, scales: tuple = (1.0, 1.0), next_w: Optional[torch.Tensor] = None,
+                        ids: Optional[torch.Tensor] = None):
+    """x <- x + L(u) * w with L(v) = (v - mean) / sqrt(variance + eps), u = scales[0] * y + scales[1] * y2 (activation
+    tensors, row-strided; y2 may be None) or the `RoutedRows` / fp32 sum of a routed mixture. Returns (x, n): n = x, or
+    L(x) * next_w, as `out_dtype` (x itself where that is float32 and there is no next_w). x fp32 [T, W], in place.
+    `ids`: y is an embedding table, u = y[ids] (zero rows for ids outside it) and x = L(u) * w is new (x None)."""
+    routed, y3 = None, None
+    if isinstance(y, RoutedRows):
+        y, y3, routed = None, y.y, (y if y.dest is not None else None)
+    W = w.numel()
+    T = ids.shape[0] if ids is not None else x.shape[0]
+    assert (x is None) == (ids is not None)
+
+    def ln(v):
+        c = v - v.mean(-1, keepdim=True)
+        return c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps)
+    if not native_device(w):
+        if ids is not None:
+            u = embed_rows(ids, y)
+        elif routed is not None:
+            rows = y3[routed.dest.long()]
+            u = (rows * routed.wts[:, :, None]).sum(1) if routed.wts is not None else rows.sum(1)
+        elif y3 is not None:
+            u = y3
+        else:
+            u = scales[0] * y.float() + (scales[1] * y2.float() if y2 is not None else 0.0)
+        x = ln(u) * w if x is None else x.add_(ln(u) * w)
+        return x, ((ln(x) * next_w).to(out_dtype) if next_w is not None else x.to(out_dtype))
+    if x is None:
+        assert y.dim() == 2 and y.is_contiguous() and y.shape[1] == W
+        x = torch.empty(T, W, dtype=torch.float32, device=w.device)
+    assert x.dtype == torch.float32 and x.is_contiguous() and x.shape[1] == W
+    for t in (w, next_w):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == W)
+    if ids is None:
+        for t in (y, y2):
+            assert t is None or (t.stride(1) == 1 and t.shape == x.shape and t.dtype == y.dtype)
+    assert y3 is None or (y3.dtype == torch.float32 and y3.is_contiguous() and y3.shape[1] == W)
+    if routed is not None:
+        assert routed.dest.dtype == torch.int32 and routed.dest.is_contiguous() and routed.dest.shape[0] == T
+        assert routed.wts is None or (routed.wts.is_contiguous() and routed.wts.shape == routed.dest.shape)
+    else:
+        assert y3 is None or y3.shape[0] == T
+    alias = out_dtype == torch.float32 and next_w is None
+    out = None if alias else torch.empty(T, W, dtype=out_dtype, device=x.device)
+    mixers().layer_norm_residual(x.data_ptr(), _p(y), y.stride(0) if y is not None else 0, float(scales[0]), _p(y2),
+                                 y2.stride(0) if y2 is not None else 0, float(scales[1]), is_f32(y) if y is not None else True,
+                                 _i32(ids).data_ptr() if ids is not None else 0, y.shape[0] if ids is not None else 0, _p(y3),
+                                 _p(routed.dest) if routed else 0, _p(routed.wts) if routed else 0,
+                                 routed.dest.shape[1] if routed else 0, w.data_ptr(), _p(next_w), float(eps), _p(out),
+                                 is_f32(out) if out is not None else True, T, W, stream_ptr())
+    return x, (x if alias else out)
+
+
+# ---------------------------------------------------------------------------- retention, time mixing
+def rotate_qk(proj: torch.Tensor, off_q: int, off_k: int, H: int, dk: int, rot: Optional[torch.Tensor], rot_dims: int,
+              k_scale: float, sm: SeqMeta):
+    """q and k of a fused projection row: the first rot_dims entries of each head rotated in (i, i + rot_dims / 2) pairs by
+    the token's position (rot_dims 0: none), k times k_scale. Returns (q, k), fp32 [T, H dk]."""
+    T, n = proj.shape[0], H * dk
+    if not native_device(proj):
+        def turn(v):
+            v = v.float().reshape(T, H, dk)
+            return (_rotate_pairs(v, rot, sm.positions, rot_dims, True) if rot_dims else v).reshape(T, n)
+        return turn(proj[:, off_q:off_q + n]), turn(proj[:, off_k:off_k + n]) * k_scale
+    assert proj.stride(1) == 1
+    assert rot_dims == 0 or (rot.dtype == torch.float32 and rot.is_contiguous() and rot.shape[1] * 2 == rot_dims)
+    out = torch.empty(2, T, n, dtype=torch.float32, device=proj.device)
+    mixers().rotate_qk(proj.data_ptr(), is_f32(proj), proj.stride(0), off_q, off_k, H, dk, _p(rot) if rot_dims else 0,
+                       rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale), _i32(sm.positions).data_ptr(),
+                       out[0].data_ptr(), out[1].data_ptr(), T, stream_ptr())
+    return out[0], out[1]
+
+
+def token_shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, sm: SeqMeta, out_dtype: torch.dtype):
+    """Mixes of every row with the previous token's, x_t + (x_(t-1) - x_t) * mu[j] for each of n vectors mu[j] (x_(-1) = 0
+    at a sequence's start): x fp32 [T, W], mu fp32 [n, W] -> [n, T, W]. state fp32 [slots, W] holds each sequence's last
+    row and is updated."""
+    T, W = x.shape
+    n = mu.shape[0]
+    out = torch.empty(n, T, W, dtype=out_dtype, device=x.device)
+    if native_device(x):
+        assert x.dtype == torch.float32 and x.is_contiguous() and mu.dtype == torch.float32 and mu.is_contiguous()
+        assert mu.shape[1] == W and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == W
+        mixers().token_shift_mix(x.data_ptr(), mu.data_ptr(), n, state.data_ptr(), _i32(sm.qsl).data_ptr(),
+                                 _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(), _i32(sm.token_seq).data_ptr(),
+                                 out.data_ptr(), is_f32(out), T, W, stream_ptr())
+        return out
+    prev = torch.zeros_like(x)
+    prev[1:] = x[:-1]
+    qsl, sl, slots = sm.qsl.tolist(), sm.seq_lens.tolist(), sm.slots.tolist()
+    for s in range(sm.num_seqs):
+        lo, hi = qsl[s], qsl[s + 1]
+        if slots[s] < 0 or hi <= lo:
+            continue
+        prev[lo] = state[slots[s]] if sl[s] > hi - lo else 0.0
+        state[slots[s]] = x[hi - 1]
+    return (x[None] + (prev - x)[None] * mu[:, None, :]).to(out_dtype)
+
+
+def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.Tensor):
+    """(r, exp(-exp(z + w0)), k) as fp32 [T, n]: the inputs of gated_linear_scan with a data-dependent decay per key
+    channel. r, k, z row-strided activation tensors; w0 fp32 [n]."""
+    T, n = r.shape
+    if not native_device(r):
+        return r.float(), torch.exp(-torch.exp(z.float() + w0)), k.float()
+    assert r.dtype == k.dtype == z.dtype and all(t.stride(1) == 1 for t in (r, k, z)) and w0.dtype == torch.float32
+    out = torch.empty(3, T, n, dtype=torch.float32, device=r.device)
+    mixers().time_mix_gates(r.data_ptr(), r.stride(0), k.data_ptr(), k.stride(0), z.data_ptr(), z.stride(0), is_f32(r),
+                            w0.data_ptr(), n, out[0].data_ptr(), out[1].data_ptr(), out[2].data_ptr(), T, stream_ptr())
+    return out[0], out[1], out[2]
+
+
+def _recurrent_step(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=None, w0=None, bonus=None, rot=None, rot_dims=0,
+                    k_scale=1.0):
+    """A step of single tokens: recurrence, per-head norm and gate in one kernel. Returns [T, H dv]."""
+    assert all(t.stride(1) == 1 and t.dtype == q.dtype for t in (q, k, v, g)) and (z is None or (z.stride(1) == 1 and z.dtype == q.dtype))
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, dk, dv)
+    out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    mixers().recurrent_step(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), g.data_ptr(),
+                            g.stride(0), _p(z), z.stride(0) if z is not None else 0, is_f32(q), _p(decay), _p(w0), _p(bonus),
+                            _p(rot) if rot_dims else 0, rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale), _p(norm_w),
+                            float(eps), state.data_ptr(), _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(),
+                            _i32(sm.positions).data_ptr(), out.data_ptr(), q.shape[0], H, dk, dv, stream_ptr())
+    return out
+
+
+# XGS_TUNE recurrent_step=0: steps of single tokens through the scan kernels too (A/B and tests)
+RECURRENT_STEP = tune.get_bool("recurrent_step", True)
+
+
+def retention(proj: torch.Tensor, H: int, dk: int, dv: int, decay: torch.Tensor, rot: Optional[torch.Tensor], rot_dims: int,
+              eps: float, state: torch.Tensor, sm: SeqMeta) -> torch.Tensor:
+    """Linear attention with one constant decay per head on the columns [q | k | v | g] of a fused projection row:
+    q, k rotated (rotate_qk), k * dk^(-1/2); S <- decay_h S + k v^T, o = S^T q; each head's o divided by its own root mean
+    square, times silu(g). state fp32 [slots, H, dk, dv]. Returns [T, H dv]."""
+    n, nv = H * dk, H * dv
+    v, g = proj[:, 2 * n:2 * n + nv], proj[:, 2 * n + nv:2 * n + 2 * nv]
+    if native_device(proj) and RECURRENT_STEP and sm.max_q == 1 and proj.shape[0] == sm.num_seqs:
+        return _recurrent_step(proj[:, :n], proj[:, n:2 * n], v, g, None, H, dk, dv, state, sm, None, eps, decay=decay, rot=rot,
+                               rot_dims=rot_dims, k_scale=dk ** -0.5)
+    q, k = rotate_qk(proj, 0, n, H, dk, rot, rot_dims, dk ** -0.5, sm)
+    o = gated_linear_scan(q, None, k, v, state, H, dk, dv, sm, decay=decay)
+    return gated_group_norm(o, g, None, eps, H, proj.dtype, gate_after=True)
+
+
+def time_mix(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, z: torch.Tensor, w0: torch.Tensor,
+             bonus: torch.Tensor, norm_w: torch.Tensor, eps: float, H: int, dk: int, dv: int, state: torch.Tensor,
+             sm: SeqMeta) -> torch.Tensor:
+    """Per head, with the decay w = exp(-exp(z + w0)) per key channel: o = (S + diag(u) k v^T)^T r with the bonus u for the
+    current token, then S <- diag(w) S + k v^T; each head's o divided by its own root mean square, times norm_w, times
+    silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided activations); state fp32 [slots, H, dk, dv]. Returns [T, H dv]."""
+    if native_device(r) and RECURRENT_STEP and sm.max_q == 1 and r.shape[0] == sm.num_seqs:
+        return _recurrent_step(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
+    q, f, kk = time_mix_gates(r, k, z, w0)
+    o = gated_linear_scan(q, f, kk, v, state, H, dk, dv, sm, bonus=bonus)
+    return gated_group_norm(o, g, norm_w, eps, H, r.dtype, gate_after=True)
