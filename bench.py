@@ -97,6 +97,12 @@ def parse():
                          "batch, --steps, --warmup, --dofivik-prompts, --dofivik-context apply)")
     ap.add_argument("--taritar-sizes", default="1b-class,8b-class")
     ap.add_argument("--taritar-only", default=None, choices=["taritar", "mixtral", "llama"])
+    ap.add_argument("--bazurax", action="store_true",
+                    help="instead of the headline: prefill and decode tokens/s of Bazurax beside Lotelix, a Mixtral-type "
+                         "model and a Llama of equal layer sizes (bench/bazurax_bench.py; --prompt-len, --concurrency = "
+                         "decode batch, --steps, --warmup, --dofivik-prompts, --dofivik-context apply)")
+    ap.add_argument("--bazurax-sizes", default="1b-class,8b-class")
+    ap.add_argument("--bazurax-only", default=None, choices=["bazurax", "lotelix", "mixtral", "llama"])
     return ap.parse_args()
 
 
@@ -191,12 +197,12 @@ def preflight(st, world: int, tp: int, dev, eng) -> dict:
 
 def main():
     a = parse()
-    if a.dofivik or a.vizonex or a.loluzen or a.lotelix or a.taritar:
+    if a.dofivik or a.vizonex or a.loluzen or a.lotelix or a.taritar or a.bazurax:
         import importlib.util
         here = os.path.dirname(os.path.abspath(__file__))
         sys.path.insert(0, here)
         which = "dofivik_bench" if a.dofivik else "vizonex_bench" if a.vizonex else "loluzen_bench" if a.loluzen \
-            else "lotelix_bench" if a.lotelix else "taritar_bench"
+            else "lotelix_bench" if a.lotelix else "taritar_bench" if a.taritar else "bazurax_bench"
         spec = importlib.util.spec_from_file_location(which, os.path.join(here, "bench", which + ".py"))
         mod = importlib.util.module_from_spec(spec)
         spec.loader.exec_module(mod)
