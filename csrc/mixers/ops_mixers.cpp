@@ -79,6 +79,11 @@ int recurrent_step(const void*, int64_t, const void*, int64_t, const void*, int6
 void decay_gates(const void*, bool, int64_t, int, int, int, float, const void*, int64_t, const float*, float, float*, float*,
                  float*, int, hipStream_t);
 void moe_combine(const float*, const int32_t*, const float*, int, int, int, float*, hipStream_t);
+int64_t chunk_recurrence_scratch_floats(int, int, int, int, int, int);
+int chunk_recurrence(const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
+                     int64_t, const float*, const float*, const float*, const float*, int, int, float, const float*, float,
+                     float*, const int32_t*, const int32_t*, const int32_t*, void*, float*, int, int, int, int, int, int, int,
+                     float*, hipStream_t);
 void canon_conv(const float*, const float*, float*, const int32_t*, const int32_t*, const int32_t*, void*, bool, int, int,
                 int, int, hipStream_t);
 void scaled_add_rmsnorm(const float*, const void*, bool, int64_t, const float*, float, const float*, float, float, float*,
@@ -406,6 +411,26 @@ PYBIND11_MODULE(_mixers, m) {
                                  P<const float>(norm_w), eps, P<float>(state), P<const int32_t>(sl), P<const int32_t>(slots),
                                  P<const int32_t>(pos), P<void>(out), ns, H, dk, dv, S(st));
     check(rc, "recurrent_step");
+  });
+  m.def("chunk_recurrence_scratch_floats", [](int T, int ns, int H, int dk, int dv, int seg) {
+    if (seg < 1) throw std::invalid_argument("chunk_recurrence: segments must be positive");
+    return xgm::chunk_recurrence_scratch_floats(T, ns, H, dk, dv, seg);
+  });
+  m.def("chunk_recurrence", [](uintptr_t q, int64_t ld_q, uintptr_t k, int64_t ld_k, uintptr_t v, int64_t ld_v, uintptr_t g,
+                               int64_t ld_g, uintptr_t z, int64_t ld_z, uintptr_t decay, uintptr_t w0, uintptr_t bonus,
+                               uintptr_t rot, int rot_rows, int rot_dims, float k_scale, uintptr_t norm_w, float eps,
+                               uintptr_t state, uintptr_t qsl, uintptr_t sl, uintptr_t slots, uintptr_t out, uintptr_t o32,
+                               int ns, int max_q, int T, int H, int dk, int dv, int seg, uintptr_t scratch, uintptr_t st) {
+    const int64_t nk = (int64_t)H * dk, nv = (int64_t)H * dv;
+    if (ld_q < nk || ld_k < nk || ld_v < nv || (g && ld_g < nv) || (z && ld_z < nk) || rot_dims < 0)
+      throw std::invalid_argument("chunk_recurrence: inconsistent sizes");
+    int rc = xgm::chunk_recurrence(P<const void>(q), ld_q, P<const void>(k), ld_k, P<const void>(v), ld_v, P<const void>(g),
+                                   ld_g, P<const void>(z), ld_z, P<const float>(decay), P<const float>(w0),
+                                   P<const float>(bonus), P<const float>(rot), rot_rows, rot_dims, k_scale,
+                                   P<const float>(norm_w), eps, P<float>(state), P<const int32_t>(qsl),
+                                   P<const int32_t>(sl), P<const int32_t>(slots), P<void>(out), P<float>(o32), ns, max_q, T,
+                                   H, dk, dv, seg, P<float>(scratch), S(st));
+    check(rc, "chunk_recurrence");
   });
   m.def("canon_conv", [](uintptr_t x, uintptr_t w, uintptr_t state, uintptr_t qsl, uintptr_t sl, uintptr_t slots,
                          uintptr_t out, bool out_f32, int ns, int max_q, int W, int taps, uintptr_t st) {

@@ -152,3 +152,82 @@ def forward(cfg, w, tokens, keep=None):
         if keep is not None:
             keep.append(x.clone())
     return layer_norm(x, d(w["final.norm"]), eps) @ d(w["embed"]).T
+
+
+def random_weights(cfg, seed=0):
+    """Random weights of a configuration, rounded to bfloat16 (what a checkpoint stores). `decay_rank` of a right branch
+    (the rank of its decay projection) is read from the mixer's dictionary and not written to config.json."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+    out = {}
+
+    def mat(name, o, i, gain=1.0):
+        out[name] = torch.randn(o, i, generator=g) * gain / math.sqrt(i)
+
+    def vec(name, n, std, mean=0.0):
+        out[name] = torch.randn(n, generator=g) * std + mean
+    out["embed"] = torch.randn(V, W, generator=g) * 0.5
+    vec("embed.norm", W, 0.2, 1.0)
+    vec("final.norm", W, 0.2, 1.0)
+    for n, L in enumerate(cfg["layers"]):
+        pre, m = f"l{n}.", L["mixer"]
+        vec(pre + "norm1", W, 0.2, 0.7)
+        if L["type"] == "retention":
+            H, dk, dv = m["heads"], m["dim"], m["vdim"]
+            for nm, rows in (("q", H * dk), ("k", H * dk), ("v", H * dv), ("g", H * dv)):
+                mat(pre + "mix." + nm, rows, W)
+            mat(pre + "mix.o", W, H * dv)
+        else:
+            a, r = m["left"], m["right"]
+            H, G, dk, dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            for nm, rows in (("q", H * dk), ("k", G * dk), ("v", G * dv), ("g", H)):
+                mat(pre + "mix.left." + nm, rows, W)
+            vec(pre + "mix.left.q.norm", H * dk, 0.3, 1.2)
+            vec(pre + "mix.left.k.norm", G * dk, 0.3, 1.2)
+            mat(pre + "mix.left.o", W, H * dv)
+            R, rk = r["heads"] * r["dim"], r.get("decay_rank", 4)
+            for s in "rkvgw":
+                out[pre + "mix.right.mu." + s] = torch.rand(W, generator=g)
+            for s in "rkvg":
+                mat(pre + "mix.right." + s, R, W)
+            mat(pre + "mix.right.w1", rk, W)
+            mat(pre + "mix.right.w2", R, rk)
+            out[pre + "mix.right.w0"] = torch.rand(R, generator=g) * 5.0 - 5.0
+            out[pre + "mix.right.u"] = torch.randn(r["heads"], r["dim"], generator=g)
+            vec(pre + "mix.right.norm", R, 0.3, 1.0)
+            mat(pre + "mix.right.o", W, R)
+        mlp = L.get("mlp")
+        if mlp is None:
+            continue
+        vec(pre + "norm2", W, 0.2, 0.7)
+
+        def ff(p, n):
+            mat(p + "gate", n, W)
+            mat(p + "up", n, W)
+            mat(p + "down", W, n)
+        if mlp["kind"] == "dense":
+            ff(pre + "mlp.", mlp["ff"])
+        else:
+            E = mlp["router"]["experts"]
+            mat(pre + "mlp.router", E, W, 2.0)
+            vec(pre + "mlp.router.b", E, 0.5)
+            for e in range(E):
+                ff(f"{pre}mlp.e{e}.", mlp["expert"]["ff"])
+    return {k: v.to(torch.bfloat16).to(F64) for k, v in out.items()}
+
+
+def write_checkpoint(path, cfg, Wt):
+    """config.json + model.safetensors (bfloat16) of a test model."""
+    import copy
+    import json
+    import os
+
+    from safetensors.torch import save_file
+    c = copy.deepcopy(cfg)
+    for L in c["layers"]:
+        if L["type"] == "parallel":
+            L["mixer"]["right"].pop("decay_rank", None)
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(c, f)
+    save_file({k: v.to(torch.bfloat16).contiguous() for k, v in Wt.items()}, os.path.join(path, "model.safetensors"))

@@ -50,6 +50,7 @@ class Retention(nn.Module):
         self.n, self.nv = self.H * self.dk, self.H * self.dv
         self.rot = m.get("rot") or None
         self.rot_dims = int(self.rot["dims"]) if self.rot else 0
+        self.decay_range = (min(float(a) for a in m["decay"]), max(float(a) for a in m["decay"]))
         self.register_buffer("decay", torch.tensor([float(a) for a in m["decay"]], dtype=torch.float32, device=device))
         self.in_proj = _p(torch.empty(2 * self.n + 2 * self.nv, width, device=device, dtype=dtype))   # rows [q | k | v | g]
         self.o = _p(torch.empty(width, self.nv, device=device, dtype=dtype))
@@ -59,7 +60,7 @@ class Retention(nn.Module):
 
     def forward(self, h, sm: sq.SeqMeta, lc: LayerCache, rot):
         y = sq.retention(F.linear(h, self.in_proj), self.H, self.dk, self.dv, self.decay, rot, self.rot_dims, self.eps,
-                         lc.gla, sm)
+                         lc.gla, sm, self.decay_range)
         return F.linear(y, self.o)
 
 

@@ -1412,16 +1412,65 @@ def _recurrent_step(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=None
 RECURRENT_STEP = tune.get_bool("recurrent_step", True)
 
 
+# XGS_TUNE chunk_recurrence=0: prompt portions through the general scan for bf16 too (A/B and tests)
+CHUNK_RECURRENCE = tune.get_bool("chunk_recurrence", True)
+CHUNK_DK = (32, 64, 96, 128, 256)   # key sizes of the matrix-core form
+CHUNK_MIN_DECAY = 2.0 ** -6         # ... and the smallest constant decay (its 16th power's inverse must stay in range)
+CHUNK_FUSE_DV = 128                 # value sizes up to which one workgroup holds a head: norm and gate inside
+CHUNK_FILL_WGS = 512                # long portions are cut into segments until about this many workgroups run ...
+CHUNK_MIN_SEG, CHUNK_MAX_SEGS = 128, 32   # ... of at least / at most this size and number
+
+
+def _chunk_segments(sm: SeqMeta, T: int, H: int, dv: int) -> int:
+    """Tokens per segment of a step's portions (max_q rounded up: one segment, no second launch)."""
+    whole = (sm.max_q + 31) // 32 * 32
+    wgs = max(1, T // sm.max_q) * H * ((dv + 127) // 128)
+    n = min(CHUNK_MAX_SEGS, CHUNK_FILL_WGS // wgs, whole // CHUNK_MIN_SEG)
+    if n <= 1:
+        return whole
+    return ((whole + n - 1) // n + 31) // 32 * 32
+
+
+def _chunk_recurrence(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=None, w0=None, bonus=None, rot=None, rot_dims=0,
+                      k_scale=1.0):
+    """Prompt portions on the matrix cores: recurrence, and per-head norm and gate in the same launch up to CHUNK_FUSE_DV
+    value columns. Returns [T, H dv]."""
+    assert all(t.stride(1) == 1 and t.dtype == torch.bfloat16 for t in (q, k, v, g)) and (z is None or (z.stride(1) == 1 and z.dtype == q.dtype))
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, dk, dv)
+    T = q.shape[0]
+    fuse = dv <= CHUNK_FUSE_DV
+    out = torch.empty(T, H * dv, dtype=torch.bfloat16 if fuse else torch.float32, device=q.device)
+    M = mixers()
+    seg = _chunk_segments(sm, T, H, dv)
+    scratch = None
+    if seg < sm.max_q:
+        scratch = torch.empty(M.chunk_recurrence_scratch_floats(T, sm.num_seqs, H, dk, dv, seg), dtype=torch.float32,
+                              device=q.device)
+    M.chunk_recurrence(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
+                       g.data_ptr() if fuse else 0, g.stride(0), _p(z), z.stride(0) if z is not None else 0, _p(decay), _p(w0),
+                       _p(bonus), _p(rot) if rot_dims else 0, rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale),
+                       _p(norm_w), float(eps), state.data_ptr(), _i32(sm.qsl).data_ptr(), _i32(sm.seq_lens).data_ptr(),
+                       _i32(sm.slots).data_ptr(), out.data_ptr() if fuse else 0, 0 if fuse else out.data_ptr(), sm.num_seqs,
+                       sm.max_q, T, H, dk, dv, seg, _p(scratch), stream_ptr())
+    return out if fuse else gated_group_norm(out, g, norm_w, eps, H, q.dtype, gate_after=True)
+
+
 def retention(proj: torch.Tensor, H: int, dk: int, dv: int, decay: torch.Tensor, rot: Optional[torch.Tensor], rot_dims: int,
-              eps: float, state: torch.Tensor, sm: SeqMeta) -> torch.Tensor:
+              eps: float, state: torch.Tensor, sm: SeqMeta, decay_range: tuple = (0.0, 1.0)) -> torch.Tensor:
     """Linear attention with one constant decay per head on the columns [q | k | v | g] of a fused projection row:
     q, k rotated (rotate_qk), k * dk^(-1/2); S <- decay_h S + k v^T, o = S^T q; each head's o divided by its own root mean
-    square, times silu(g). state fp32 [slots, H, dk, dv]. Returns [T, H dv]."""
+    square, times silu(g). state fp32 [slots, H, dk, dv]. `decay_range`: the smallest and largest decay (host floats; the
+    matrix-core form takes a limited range). Returns [T, H dv]."""
     n, nv = H * dk, H * dv
     v, g = proj[:, 2 * n:2 * n + nv], proj[:, 2 * n + nv:2 * n + 2 * nv]
     if native_device(proj) and RECURRENT_STEP and sm.max_q == 1 and proj.shape[0] == sm.num_seqs:
         return _recurrent_step(proj[:, :n], proj[:, n:2 * n], v, g, None, H, dk, dv, state, sm, None, eps, decay=decay, rot=rot,
                                rot_dims=rot_dims, k_scale=dk ** -0.5)
+    if native_device(proj) and CHUNK_RECURRENCE and proj.dtype == torch.bfloat16 and dk in CHUNK_DK and dv % 8 == 0 \
+            and rot_dims % 16 == 0 and CHUNK_MIN_DECAY <= decay_range[0] and decay_range[1] <= 1.0 and proj.stride(0) % 8 == 0 \
+            and proj.data_ptr() % 16 == 0:
+        return _chunk_recurrence(proj[:, :n], proj[:, n:2 * n], v, g, None, H, dk, dv, state, sm, None, eps, decay=decay,
+                                 rot=rot, rot_dims=rot_dims, k_scale=dk ** -0.5)
     q, k = rotate_qk(proj, 0, n, H, dk, rot, rot_dims, dk ** -0.5, sm)
     o = gated_linear_scan(q, None, k, v, state, H, dk, dv, sm, decay=decay)
     return gated_group_norm(o, g, None, eps, H, proj.dtype, gate_after=True)
@@ -1435,6 +1484,9 @@ def time_mix(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor,
     silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided activations); state fp32 [slots, H, dk, dv]. Returns [T, H dv]."""
     if native_device(r) and RECURRENT_STEP and sm.max_q == 1 and r.shape[0] == sm.num_seqs:
         return _recurrent_step(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
+    if native_device(r) and CHUNK_RECURRENCE and r.dtype == torch.bfloat16 and dk == dv and dk in CHUNK_DK and dk != 96 \
+            and all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (r, k, v, g, z)):
+        return _chunk_recurrence(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
     q, f, kk = time_mix_gates(r, k, z, w0)
     o = gated_linear_scan(q, f, kk, v, state, H, dk, dv, sm, bonus=bonus)
     return gated_group_norm(o, g, norm_w, eps, H, r.dtype, gate_after=True)
