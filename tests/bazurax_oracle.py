@@ -155,7 +155,9 @@ def forward(cfg, w, tokens, keep=None):
 
 
 def random_weights(cfg, seed=0):
-    """Random weights of a configuration, rounded to bfloat16 (what a checkpoint stores). `decay_rank` of a right branch
+    """Random weights of a configuration, rounded to bfloat16 (what a checkpoint stores). Recurrent queries and keys are
+    correlated (and the bonus is mostly positive), so that a token's own key scores clearly above zero: an output whose terms
+    almost cancel is blown up by its head norm, rounding included, and early tokens have few terms. `decay_rank` of a right branch
     (the rank of its decay projection) is read from the mixer's dictionary and not written to config.json."""
     g = torch.Generator().manual_seed(seed)
     W, V = cfg["width"], cfg["vocab"]
@@ -176,6 +178,7 @@ def random_weights(cfg, seed=0):
             H, dk, dv = m["heads"], m["dim"], m["vdim"]
             for nm, rows in (("q", H * dk), ("k", H * dk), ("v", H * dv), ("g", H * dv)):
                 mat(pre + "mix." + nm, rows, W)
+            out[pre + "mix.k"] = 0.6 * out[pre + "mix.k"] + 0.8 * out[pre + "mix.q"]
             mat(pre + "mix.o", W, H * dv)
         else:
             a, r = m["left"], m["right"]
@@ -190,10 +193,11 @@ def random_weights(cfg, seed=0):
                 out[pre + "mix.right.mu." + s] = torch.rand(W, generator=g)
             for s in "rkvg":
                 mat(pre + "mix.right." + s, R, W)
+            out[pre + "mix.right.k"] = 0.6 * out[pre + "mix.right.k"] + 0.8 * out[pre + "mix.right.r"]
             mat(pre + "mix.right.w1", rk, W)
             mat(pre + "mix.right.w2", R, rk)
             out[pre + "mix.right.w0"] = torch.rand(R, generator=g) * 5.0 - 5.0
-            out[pre + "mix.right.u"] = torch.randn(r["heads"], r["dim"], generator=g)
+            out[pre + "mix.right.u"] = torch.randn(r["heads"], r["dim"], generator=g) * 0.5 + 1.0
             vec(pre + "mix.right.norm", R, 0.3, 1.0)
             mat(pre + "mix.right.o", W, R)
         mlp = L.get("mlp")
