@@ -1417,15 +1417,17 @@ CHUNK_RECURRENCE = tune.get_bool("chunk_recurrence", True)
 CHUNK_DK = (32, 64, 96, 128, 256)   # key sizes of the matrix-core form
 CHUNK_MIN_DECAY = 2.0 ** -6         # ... and the smallest constant decay (its 16th power's inverse must stay in range)
 CHUNK_FUSE_DV = 128                 # value sizes up to which one workgroup holds a head: norm and gate inside
-CHUNK_FILL_WGS = 512                # long portions are cut into segments until about this many workgroups run ...
+CHUNK_FILL_WGS = 512                # long portions are cut into segments until about this many workgroups run (half as many
+                                    # for the large heads, one workgroup of which fills a compute unit) ...
 CHUNK_MIN_SEG, CHUNK_MAX_SEGS = 128, 32   # ... of at least / at most this size and number
 
 
-def _chunk_segments(sm: SeqMeta, T: int, H: int, dv: int) -> int:
+def _chunk_segments(sm: SeqMeta, T: int, H: int, dk: int, dv: int, time_mixing: bool) -> int:
     """Tokens per segment of a step's portions (max_q rounded up: one segment, no second launch)."""
     whole = (sm.max_q + 31) // 32 * 32
     wgs = max(1, T // sm.max_q) * H * ((dv + 127) // 128)
-    n = min(CHUNK_MAX_SEGS, CHUNK_FILL_WGS // wgs, whole // CHUNK_MIN_SEG)
+    fill = CHUNK_FILL_WGS // (2 if dk > (64 if time_mixing else 128) else 1)
+    n = min(CHUNK_MAX_SEGS, fill // wgs, whole // CHUNK_MIN_SEG)
     if n <= 1:
         return whole
     return ((whole + n - 1) // n + 31) // 32 * 32
@@ -1441,7 +1443,7 @@ def _chunk_recurrence(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=No
     fuse = dv <= CHUNK_FUSE_DV
     out = torch.empty(T, H * dv, dtype=torch.bfloat16 if fuse else torch.float32, device=q.device)
     M = mixers()
-    seg = _chunk_segments(sm, T, H, dv)
+    seg = _chunk_segments(sm, T, H, dk, dv, decay is None)
     scratch = None
     if seg < sm.max_q:
         scratch = torch.empty(M.chunk_recurrence_scratch_floats(T, sm.num_seqs, H, dk, dv, seg), dtype=torch.float32,
