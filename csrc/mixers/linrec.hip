@@ -4,8 +4,9 @@
 //   rotate_qk        q and k of a fused projection row, the first rot_dims entries of each head rotated in pairs
 //                    (i, i + rot_dims / 2) by the token's position, k times a constant; fp32 tensors
 //   token_shift_mix  n mixes x_t + (x_(t-1) - x_t) mu_s of each row with the previous token's, as activation tensors
-//                    [n][T][W]; x_(-1) comes from the slot's carried row (zeros at a sequence's start), which takes the
+//                    [n][T rounded up to whole tiles][W]; x_(-1) comes from the slot's carried row (zeros at a sequence's start), which takes the
 //                    portion's last row
+//   low_rank_decay   z = W2 tanh(W1 x) for steps of few rows, one workgroup per row, all fp32 between the weights
 //   time_mix_gates   r, k as fp32 and the decay f = exp(-exp(z + w0))
 //   recurrent_step   steps of single tokens, one workgroup per (sequence, head): rotation or decay, the state update
 //                      S <- diag(f) S + k v^T,   o = S^T q  (after the update)  or  o = (S_old + diag(u) k v^T)^T q,
@@ -50,7 +51,7 @@ __global__ __launch_bounds__(256) void token_shift_mix_kernel(const float* __res
                                                               const int32_t* __restrict__ seq_lens,
                                                               const int32_t* __restrict__ slots,
                                                               const int32_t* __restrict__ token_seq, TO* __restrict__ out,
-                                                              int T_, int W) {
+                                                              int64_t pitch, int W) {
   const int t = blockIdx.x;
   const int c = 4 * (blockIdx.y * 256 + threadIdx.x);
   if (c >= W) return;
@@ -80,7 +81,7 @@ __global__ __launch_bounds__(256) void token_shift_mix_kernel(const float* __res
   for (int j = 0; j < n; ++j) {
     float o[4];
     const float* mj = mu + (int64_t)j * W + c;
-    TO* oj = out + ((int64_t)j * T_ + t) * W + c;
+    TO* oj = out + (j * pitch + t) * W + c;
     if (quad) {
       float g[4];
       ld4(mj, g);
@@ -107,6 +108,57 @@ __global__ __launch_bounds__(256) void time_mix_gates_kernel(const T* __restrict
   fo[i] = expf(-expf(ldf(z + t * ld_z + c) + w0[c]));
 }
 
+constexpr int kMaxRank = 256;
+
+template <typename T>
+__global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict__ x, int64_t ld_x, const T* __restrict__ w1,
+                                                             const T* __restrict__ w2, int W, int rank, int n,
+                                                             float* __restrict__ z) {
+  extern __shared__ float row[];   // [W]
+  __shared__ __attribute__((aligned(16))) float th[kMaxRank];
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  for (int c = threadIdx.x; c < W; c += 256) row[c] = ldf(x + t * ld_x + c);
+  __syncthreads();
+  const bool quad = (W & 3) == 0;
+  for (int j0 = wave * 4; j0 < rank; j0 += 16) {   // four rows of W1 per wave at a time (past the last: it again, not stored)
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+    if (quad) {
+      for (int c = 4 * lane; c < W; c += 256) {
+        float a[4], b[4][4];
+        ld4(row + c, a);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ld4(w1 + (int64_t)min(j0 + j, rank - 1) * W + c, b[j]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j] += a[0] * b[j][0] + a[1] * b[j][1] + a[2] * b[j][2] + a[3] * b[j][3];
+      }
+    } else {
+      for (int c = lane; c < W; c += 64)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j] += row[c] * ldf(w1 + (int64_t)min(j0 + j, rank - 1) * W + c);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      acc[j] = wave_sum(acc[j]);
+      if (lane == 0 && j0 + j < rank) th[j0 + j] = tanhf(acc[j]);
+    }
+  }
+  __syncthreads();
+  for (int c = threadIdx.x; c < n; c += 256) {
+    const T* wr = w2 + (int64_t)c * rank;
+    float acc = 0.f;
+    if ((rank & 3) == 0) {
+      for (int j = 0; j < rank; j += 4) {
+        float b[4];
+        ld4(wr + j, b);
+        acc += th[j] * b[0] + th[j + 1] * b[1] + th[j + 2] * b[2] + th[j + 3] * b[3];
+      }
+    } else {
+      for (int j = 0; j < rank; ++j) acc += th[j] * ldf(wr + j);
+    }
+    z[(int64_t)t * n + c] = acc;
+  }
+}
+
 // ------------------------------------------------------------------ single tokens
 struct StepArgs {
   const void *q, *k, *v, *g, *z;   // head h of token t at row t: columns h dk .. / h dv ..
@@ -125,14 +177,14 @@ struct StepArgs {
 
 constexpr int kStepThreads = 256, kStepMaxDk = 256;
 
-template <typename T, int CV>
+template <typename T, typename TO, int CV>
 __global__ __launch_bounds__(kStepThreads) void recurrent_step_kernel(const StepArgs a) {
   extern __shared__ float opart[];   // [row groups][dv]
   __shared__ float qs[kStepMaxDk], ks[kStepMaxDk], fs[kStepMaxDk];
   __shared__ float red[kStepThreads / 64];
   const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int dk = a.dk, dv = a.dv, slot = a.slots[s];
-  T* out = (T*)a.out + ((int64_t)s * a.H + h) * dv;
+  TO* out = (TO*)a.out + ((int64_t)s * a.H + h) * dv;
   if (slot < 0) {   // padding row
     for (int c = tid; c < dv; c += kStepThreads) stf(out + c, 0.f);
     return;
@@ -232,11 +284,12 @@ void rotate_qk(const void* proj, bool f32, int64_t ld, int off_q, int off_k, int
 }
 
 void token_shift_mix(const float* x, const float* mu, int n, float* state, const int32_t* qsl, const int32_t* seq_lens,
-                     const int32_t* slots, const int32_t* token_seq, void* out, bool out_f32, int T_, int W, hipStream_t st) {
+                     const int32_t* slots, const int32_t* token_seq, void* out, bool out_f32, int T_, int pitch, int W,
+                     hipStream_t st) {
   if (T_ <= 0 || n <= 0) return;
   dim3 grid(T_, (W + 1023) / 1024);
   XGM_DISPATCH_T(out_f32, token_shift_mix_kernel<T><<<grid, 256, 0, st>>>(x, mu, n, state, qsl, seq_lens, slots, token_seq,
-                                                                          (T*)out, T_, W);)
+                                                                          (T*)out, pitch, W);)
 }
 
 void time_mix_gates(const void* r, int64_t ld_r, const void* k, int64_t ld_k, const void* z, int64_t ld_z, bool f32,
@@ -247,8 +300,17 @@ void time_mix_gates(const void* r, int64_t ld_r, const void* k, int64_t ld_k, co
                           (const T*)r, ld_r, (const T*)k, ld_k, (const T*)z, ld_z, w0, n, ro, fo, ko, total);)
 }
 
+int low_rank_decay(const void* x, int64_t ld_x, bool f32, const void* w1, const void* w2, int W, int rank, int n, float* z,
+                   int T_, hipStream_t st) {
+  if (T_ <= 0) return 0;
+  if (W < 1 || W > 16000 || rank < 1 || rank > kMaxRank || n < 1 || (uintptr_t)w1 % 16 || (uintptr_t)w2 % 16) return -1;
+  XGM_DISPATCH_T(f32, low_rank_decay_kernel<T><<<T_, 256, (size_t)W * sizeof(float), st>>>(
+                          (const T*)x, ld_x, (const T*)w1, (const T*)w2, W, rank, n, z);)
+  return 0;
+}
+
 int recurrent_step(const void* q, int64_t ld_q, const void* k, int64_t ld_k, const void* v, int64_t ld_v, const void* g,
-                   int64_t ld_g, const void* z, int64_t ld_z, bool f32, const float* decay, const float* w0,
+                   int64_t ld_g, const void* z, int64_t ld_z, bool f32, bool out_f32, const float* decay, const float* w0,
                    const float* bonus, const float* rot, int rot_rows, int rot_dims, float k_scale, const float* norm_w,
                    float eps, float* state, const int32_t* seq_lens, const int32_t* slots, const int32_t* positions,
                    void* out, int ns, int H, int dk, int dv, hipStream_t st) {
@@ -261,11 +323,21 @@ int recurrent_step(const void* q, int64_t ld_q, const void* k, int64_t ld_k, con
   const int cv = dv % 4 == 0 ? 4 : 1, ct = (dv + cv - 1) / cv, rg = ct < kStepThreads ? kStepThreads / ct : 1;
   const size_t lds = (size_t)rg * dv * sizeof(float);
   dim3 grid(ns, H);
-  if (cv == 4) {
-    XGM_DISPATCH_T(f32, recurrent_step_kernel<T, 4><<<grid, kStepThreads, lds, st>>>(a);)
-  } else {
-    XGM_DISPATCH_T(f32, recurrent_step_kernel<T, 1><<<grid, kStepThreads, lds, st>>>(a);)
+  if (!f32 && out_f32) return -1;
+#define XGM_RS(TI, TO)                                                          \
+  if (cv == 4) {                                                                \
+    recurrent_step_kernel<TI, TO, 4><<<grid, kStepThreads, lds, st>>>(a);       \
+  } else {                                                                      \
+    recurrent_step_kernel<TI, TO, 1><<<grid, kStepThreads, lds, st>>>(a);       \
   }
+  if (!f32) {
+    XGM_RS(bf16, bf16)
+  } else if (out_f32) {
+    XGM_RS(float, float)
+  } else {
+    XGM_RS(float, bf16)
+  }
+#undef XGM_RS
   return 0;
 }
 

@@ -70,11 +70,12 @@ int layer_norm_residual(float*, const void*, int64_t, float, const void*, int64_
 void rotate_qk(const void*, bool, int64_t, int, int, int, int, const float*, int, int, float, const int32_t*, float*, float*,
                int, hipStream_t);
 void token_shift_mix(const float*, const float*, int, float*, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
-                     void*, bool, int, int, hipStream_t);
+                     void*, bool, int, int, int, hipStream_t);
+int low_rank_decay(const void*, int64_t, bool, const void*, const void*, int, int, int, float*, int, hipStream_t);
 void time_mix_gates(const void*, int64_t, const void*, int64_t, const void*, int64_t, bool, const float*, int, float*, float*,
                     float*, int, hipStream_t);
 int recurrent_step(const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
-                   int64_t, bool, const float*, const float*, const float*, const float*, int, int, float, const float*,
+                   int64_t, bool, bool, const float*, const float*, const float*, const float*, int, int, float, const float*,
                    float, float*, const int32_t*, const int32_t*, const int32_t*, void*, int, int, int, int, hipStream_t);
 void decay_gates(const void*, bool, int64_t, int, int, int, float, const void*, int64_t, const float*, float, float*, float*,
                  float*, int, hipStream_t);
@@ -382,13 +383,20 @@ PYBIND11_MODULE(_mixers, m) {
     check(0, "rotate_qk");
   });
   m.def("token_shift_mix", [](uintptr_t x, uintptr_t mu, int n, uintptr_t state, uintptr_t qsl, uintptr_t sl,
-                              uintptr_t slots, uintptr_t token_seq, uintptr_t out, bool out_f32, int T, int W,
+                              uintptr_t slots, uintptr_t token_seq, uintptr_t out, bool out_f32, int T, int pitch, int W,
                               uintptr_t st) {
-    if (n < 1 || W < 1) throw std::invalid_argument("token_shift_mix: inconsistent sizes");
+    if (n < 1 || W < 1 || pitch < T) throw std::invalid_argument("token_shift_mix: inconsistent sizes");
     xgm::token_shift_mix(P<const float>(x), P<const float>(mu), n, P<float>(state), P<const int32_t>(qsl),
                          P<const int32_t>(sl), P<const int32_t>(slots), P<const int32_t>(token_seq), P<void>(out), out_f32,
-                         T, W, S(st));
+                         T, pitch, W, S(st));
     check(0, "token_shift_mix");
+  });
+  m.def("low_rank_decay", [](uintptr_t x, int64_t ld_x, bool f32, uintptr_t w1, uintptr_t w2, int W, int rank, int n,
+                             uintptr_t z, int T, uintptr_t st) {
+    if (ld_x < W) throw std::invalid_argument("low_rank_decay: row stride below the width");
+    int rc = xgm::low_rank_decay(P<const void>(x), ld_x, f32, P<const void>(w1), P<const void>(w2), W, rank, n, P<float>(z),
+                                 T, S(st));
+    check(rc, "low_rank_decay");
   });
   m.def("time_mix_gates", [](uintptr_t r, int64_t ld_r, uintptr_t k, int64_t ld_k, uintptr_t z, int64_t ld_z, bool f32,
                              uintptr_t w0, int n, uintptr_t ro, uintptr_t fo, uintptr_t ko, int T, uintptr_t st) {
@@ -398,15 +406,15 @@ PYBIND11_MODULE(_mixers, m) {
     check(0, "time_mix_gates");
   });
   m.def("recurrent_step", [](uintptr_t q, int64_t ld_q, uintptr_t k, int64_t ld_k, uintptr_t v, int64_t ld_v, uintptr_t g,
-                             int64_t ld_g, uintptr_t z, int64_t ld_z, bool f32, uintptr_t decay, uintptr_t w0,
-                             uintptr_t bonus, uintptr_t rot, int rot_rows, int rot_dims, float k_scale, uintptr_t norm_w,
+                             int64_t ld_g, uintptr_t z, int64_t ld_z, bool f32, bool out_f32, uintptr_t decay,
+                             uintptr_t w0, uintptr_t bonus, uintptr_t rot, int rot_rows, int rot_dims, float k_scale, uintptr_t norm_w,
                              float eps, uintptr_t state, uintptr_t sl, uintptr_t slots, uintptr_t pos, uintptr_t out, int ns,
                              int H, int dk, int dv, uintptr_t st) {
     const int64_t nk = (int64_t)H * dk, nv = (int64_t)H * dv;
     if (ld_q < nk || ld_k < nk || ld_v < nv || ld_g < nv || (z && ld_z < nk) || rot_dims < 0 || (rot_dims && rot_rows < 1))
       throw std::invalid_argument("recurrent_step: inconsistent sizes");
     int rc = xgm::recurrent_step(P<const void>(q), ld_q, P<const void>(k), ld_k, P<const void>(v), ld_v, P<const void>(g),
-                                 ld_g, P<const void>(z), ld_z, f32, P<const float>(decay), P<const float>(w0),
+                                 ld_g, P<const void>(z), ld_z, f32, out_f32, P<const float>(decay), P<const float>(w0),
                                  P<const float>(bonus), P<const float>(rot), rot_rows, rot_dims, k_scale,
                                  P<const float>(norm_w), eps, P<float>(state), P<const int32_t>(sl), P<const int32_t>(slots),
                                  P<const int32_t>(pos), P<void>(out), ns, H, dk, dv, S(st));

@@ -596,7 +596,7 @@ def _window_case(device, dtype, H, G, dk, dv, bs, T, size, single, strong=None):
     for ctx, n in ([(0, T)] if not single else [(0, T - 6)] + [(T - 6 + i, 1) for i in range(6)]):
         sm = seq_meta(device, [(0, ctx, n)], bs, [pages])
         src = torch.cat([q[ctx:ctx + n].reshape(n, -1), k[ctx:ctx + n].reshape(n, -1), v[ctx:ctx + n].reshape(n, -1)], 1)
-        qq = sq.qk_norm_cache(src.to(dt).to(device), H * dk, G * dk, G * dv, f32(wq), f32(wk), eps, sm, kc, vc)
+        qq = sq.head_norm_rope_cache(src.to(dt).to(device), H, G, dk, dv, f32(wq), f32(wk), eps, None, 0, sm, kc, vc, dt, whole=True)
         out.append(sq.masked_attention(qq, kc, vc, H, G, dk, dv, sq.MASK_WINDOW, size, scale, None, None, bs, sm,
                                        gate=gate[ctx:ctx + n].to(dt).to(device)))
     return torch.cat(out).float().cpu().reshape(T, H * dv), ref.reshape(T, H * dv)
@@ -624,6 +624,35 @@ def test_window_edge_one_standing_out_key(device, dtype, size, edge, single):
     got, ref = _window_case(device, dtype, 4, 2, 32, 16, 16, T, size, single, strong=(T - 1, T - 1 - back))
     assert rel_err(got[-1:], ref[-1:]) < (1e-4 if dtype == "float32" else 5e-2)
     assert rel_err(got, ref) < (1e-4 if dtype == "float32" else 5e-2)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("T", [1, 7, 16, 17, 33, 64])
+@pytest.mark.parametrize("G,K,N", [(4, 64, 32), (4, 96, 48), (3, 256, 80)])
+def test_stacked_products_of_short_steps(T, G, K, N):
+    """Products with an input and a weight of their own each, in one launch; rows past the step are left alone."""
+    g = torch.Generator().manual_seed(T + K)
+    w = torch.randn(G, N, K, generator=g).to(torch.bfloat16).cuda()
+    tile = sq.stacked_tile(T, K, N, w)
+    R = (T + tile - 1) // tile * tile
+    x = torch.randn(G, R, K, generator=g).to(torch.bfloat16).cuda()
+    y = sq.stacked_linear(x, w, T)
+    ref = torch.stack([x[i].cpu().to(F64) @ w[i].cpu().to(F64).T for i in range(G)])
+    assert y.shape == (G, R, N) and float((y[:, :T].cpu().to(F64) - ref[:, :T]).abs().max()) < 1e-4 * float(ref.abs().max())
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("T,W,rank,n", [(1, 50, 1, 16), (7, 64, 6, 60), (64, 130, 16, 40), (64, 512, 64, 256), (5, 33, 130, 300),
+                                        (90, 64, 8, 64)])
+def test_low_rank_decay(device, dtype, T, W, rank, n):
+    dt = getattr(torch, dtype)
+    g = torch.Generator().manual_seed(T + W)
+    wide = bf(torch.randn(T, W + 6, generator=g))
+    w1, w2 = bf(torch.randn(rank, W, generator=g) / W ** 0.5), bf(torch.randn(n, rank, generator=g) / rank ** 0.5)
+    d = lambda t: t.to(dt).to(device)  # noqa: E731
+    z = sq.low_rank_decay(d(wide)[:, :W], d(w1), d(w2))
+    ref = torch.tanh(wide[:, :W] @ w1.T) @ w2.T
+    assert float((z.cpu().to(F64) - ref).abs().max()) < (1e-5 if dtype == "float32" else 3e-2) * float(ref.abs().max())
 
 
 @pytest.mark.parametrize("device", OP_CASES)

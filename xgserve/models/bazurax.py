@@ -80,7 +80,8 @@ class WholeNormWindowAttention(nn.Module):
 
     def forward(self, h, sm: sq.SeqMeta, lc: LayerCache, block_size: int):
         proj = F.linear(h, self.in_proj)
-        q = sq.qk_norm_cache(proj[:, :self.ch], self.nq, self.nk, self.nv, self.q_norm, self.k_norm, self.eps, sm, lc.k, lc.v)
+        q = sq.head_norm_rope_cache(proj, self.H, self.G, self.dk, self.dv, self.q_norm, self.k_norm, self.eps, None, 0, sm,
+                                    lc.k, lc.v, h.dtype, whole=True)
         o = sq.masked_attention(q, lc.k, lc.v, self.H, self.G, self.dk, self.dv, self.mask, self.size, self.scale, None, None,
                                 block_size, sm, gate=proj[:, self.ch:])
         return F.linear(o, self.o)
@@ -101,10 +102,16 @@ class TimeMix(nn.Module):
 
     def forward(self, x, sm: sq.SeqMeta, lc: LayerCache, dtype):
         """x: the fp32 mixer input (the mixes are formed before they are rounded)."""
-        mixed = sq.token_shift_mix(x, self.mu, lc.shift, sm, dtype)
-        r, k, v, g = (F.linear(mixed[j], self.rkvg[j]) for j in range(4))
-        z = F.linear(sq.tanh_cols(F.linear(mixed[4], self.w1), 0, self.rank), self.w2)
-        y = sq.time_mix(r, k, v, g, z, self.w0, self.u, self.norm, self.eps, self.H, self.dk, self.dk, lc.gla, sm)
+        T = x.shape[0]
+        tile = sq.stacked_tile(T, x.shape[1], self.n, self.rkvg) if sm.max_q == 1 else 0
+        mixed = sq.token_shift_mix(x, self.mu, lc.shift, sm, dtype, tile or 1)
+        if tile:   # single tokens: the four products in one launch
+            r, k, v, g = sq.stacked_linear(mixed[:4], self.rkvg, T)[:, :T].unbind(0)
+        else:
+            r, k, v, g = (F.linear(mixed[j], self.rkvg[j]) for j in range(4))
+        z = sq.low_rank_decay(mixed[4][:T], self.w1, self.w2)
+        y = sq.time_mix(r, k, v, g, z.to(r.dtype), self.w0, self.u, self.norm, self.eps, self.H, self.dk, self.dk, lc.gla, sm,
+                        dtype)
         return F.linear(y, self.o)
 
 

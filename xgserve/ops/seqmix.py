@@ -1355,19 +1355,22 @@ def rotate_qk(proj: torch.Tensor, off_q: int, off_k: int, H: int, dk: int, rot: 
     return out[0], out[1]
 
 
-def token_shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, sm: SeqMeta, out_dtype: torch.dtype):
+def token_shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, sm: SeqMeta, out_dtype: torch.dtype,
+                    tile: int = 1):
     """Mixes of every row with the previous token's, x_t + (x_(t-1) - x_t) * mu[j] for each of n vectors mu[j] (x_(-1) = 0
-    at a sequence's start): x fp32 [T, W], mu fp32 [n, W] -> [n, T, W]. state fp32 [slots, W] holds each sequence's last
+    at a sequence's start): x fp32 [T, W], mu fp32 [n, W] -> [n, T rounded up to whole tiles of rows, W] (rows past T are not
+    written). state fp32 [slots, W] holds each sequence's last
     row and is updated."""
     T, W = x.shape
     n = mu.shape[0]
-    out = torch.empty(n, T, W, dtype=out_dtype, device=x.device)
+    pitch = (T + tile - 1) // tile * tile
+    out = torch.empty(n, pitch, W, dtype=out_dtype, device=x.device)
     if native_device(x):
         assert x.dtype == torch.float32 and x.is_contiguous() and mu.dtype == torch.float32 and mu.is_contiguous()
         assert mu.shape[1] == W and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == W
         mixers().token_shift_mix(x.data_ptr(), mu.data_ptr(), n, state.data_ptr(), _i32(sm.qsl).data_ptr(),
                                  _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(), _i32(sm.token_seq).data_ptr(),
-                                 out.data_ptr(), is_f32(out), T, W, stream_ptr())
+                                 out.data_ptr(), is_f32(out), T, pitch, W, stream_ptr())
         return out
     prev = torch.zeros_like(x)
     prev[1:] = x[:-1]
@@ -1378,7 +1381,55 @@ def token_shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, sm: 
             continue
         prev[lo] = state[slots[s]] if sl[s] > hi - lo else 0.0
         state[slots[s]] = x[hi - 1]
-    return (x[None] + (prev - x)[None] * mu[:, None, :]).to(out_dtype)
+    out[:, :T] = (x[None] + (prev - x)[None] * mu[:, None, :]).to(out_dtype)
+    return out
+
+
+STACKED_MAX_ROWS = 64   # steps of up to this many rows run products with inputs of their own as one launch
+_STACKED_LAYOUT = {}
+
+
+def stacked_tile(T: int, K: int, N: int, w: torch.Tensor) -> int:
+    """Rows per tile of stacked_linear for steps of T rows, 0 where separate matrix products are used."""
+    if not (native_device(w) and MOE_MFMA and w.dtype == torch.bfloat16 and T <= STACKED_MAX_ROWS and K % 32 == 0 and N % 16 == 0):
+        return 0
+    return 16 if T <= 16 else 32
+
+
+def stacked_linear(x: torch.Tensor, w: torch.Tensor, T: int) -> torch.Tensor:
+    """y[g] = x[g] w[g]^T for each of G inputs with a weight of its own, in one launch on the grouped GEMM: x [G, rows, K]
+    (rows: T rounded up to stacked_tile), w [G, N, K]. Returns fp32 [G, rows, N] (rows past T are not written)."""
+    G, R, K = x.shape
+    N = w.shape[1]
+    tm = stacked_tile(T, K, N, w)
+    assert tm and R % tm == 0 and x.is_contiguous() and w.is_contiguous() and x.dtype == w.dtype
+    key = (x.device, G, R, T, tm)
+    if key not in _STACKED_LAYOUT:   # sorted layout of the grouped GEMM: group g owns rows g R .. g R + T - 1
+        i = torch.arange(G * R, dtype=torch.int32)
+        rows = torch.where(i % R < T, i, -torch.ones_like(i))
+        _STACKED_LAYOUT[key] = (rows.to(x.device), (torch.arange(G * R // tm, dtype=torch.int32) * tm // R).to(x.device))
+    rows, tile_g = _STACKED_LAYOUT[key]
+    y = torch.empty(G, R, N, dtype=torch.float32, device=x.device)
+    mixers().grouped_gemm(x.data_ptr(), False, K, w.data_ptr(), rows.data_ptr(), tile_g.data_ptr(), G * R, tm, 1, N, K, 0,
+                          y.data_ptr(), 0, 0.0, 0.0, 0, True, stream_ptr())
+    return y
+
+
+LOW_RANK_MAX_ROWS, LOW_RANK_MAX = 64, 256   # steps and ranks of the one-launch form
+
+
+def low_rank_decay(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor) -> torch.Tensor:
+    """w2 tanh(w1 x): x [T, W] row-strided activations, w1 [rank, W], w2 [n, rank]. Short steps on the GPU: one launch, fp32
+    [T, n]; else two matrix products, in the activation dtype."""
+    T, W = x.shape
+    rank, n = w1.shape[0], w2.shape[0]
+    if native_device(x) and T <= LOW_RANK_MAX_ROWS and rank <= LOW_RANK_MAX:
+        assert x.stride(1) == 1 and x.dtype == w1.dtype == w2.dtype and w1.is_contiguous() and w2.is_contiguous()
+        z = torch.empty(T, n, dtype=torch.float32, device=x.device)
+        mixers().low_rank_decay(x.data_ptr(), x.stride(0), is_f32(x), w1.data_ptr(), w2.data_ptr(), W, rank, n, z.data_ptr(),
+                                T, stream_ptr())
+        return z
+    return torch.nn.functional.linear(tanh_cols(torch.nn.functional.linear(x, w1), 0, rank), w2)
 
 
 def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.Tensor):
@@ -1386,6 +1437,7 @@ def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.
     channel. r, k, z row-strided activation tensors; w0 fp32 [n]."""
     T, n = r.shape
     if not native_device(r):
+        r, k = r.contiguous(), k.contiguous()
         return r.float(), torch.exp(-torch.exp(z.float() + w0)), k.float()
     assert r.dtype == k.dtype == z.dtype and all(t.stride(1) == 1 for t in (r, k, z)) and w0.dtype == torch.float32
     out = torch.empty(3, T, n, dtype=torch.float32, device=r.device)
@@ -1395,14 +1447,14 @@ def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.
 
 
 def _recurrent_step(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=None, w0=None, bonus=None, rot=None, rot_dims=0,
-                    k_scale=1.0):
+                    k_scale=1.0, out_dtype=None):
     """A step of single tokens: recurrence, per-head norm and gate in one kernel. Returns [T, H dv]."""
     assert all(t.stride(1) == 1 and t.dtype == q.dtype for t in (q, k, v, g)) and (z is None or (z.stride(1) == 1 and z.dtype == q.dtype))
     assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, dk, dv)
-    out = torch.empty(q.shape[0], H * dv, dtype=q.dtype, device=q.device)
+    out = torch.empty(q.shape[0], H * dv, dtype=out_dtype or q.dtype, device=q.device)
     mixers().recurrent_step(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), g.data_ptr(),
-                            g.stride(0), _p(z), z.stride(0) if z is not None else 0, is_f32(q), _p(decay), _p(w0), _p(bonus),
-                            _p(rot) if rot_dims else 0, rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale), _p(norm_w),
+                            g.stride(0), _p(z), z.stride(0) if z is not None else 0, is_f32(q), is_f32(out), _p(decay), _p(w0),
+                            _p(bonus), _p(rot) if rot_dims else 0, rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale), _p(norm_w),
                             float(eps), state.data_ptr(), _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(),
                             _i32(sm.positions).data_ptr(), out.data_ptr(), q.shape[0], H, dk, dv, stream_ptr())
     return out
@@ -1480,12 +1532,16 @@ def retention(proj: torch.Tensor, H: int, dk: int, dv: int, decay: torch.Tensor,
 
 def time_mix(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, z: torch.Tensor, w0: torch.Tensor,
              bonus: torch.Tensor, norm_w: torch.Tensor, eps: float, H: int, dk: int, dv: int, state: torch.Tensor,
-             sm: SeqMeta) -> torch.Tensor:
+             sm: SeqMeta, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
     """Per head, with the decay w = exp(-exp(z + w0)) per key channel: o = (S + diag(u) k v^T)^T r with the bonus u for the
     current token, then S <- diag(w) S + k v^T; each head's o divided by its own root mean square, times norm_w, times
-    silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided activations); state fp32 [slots, H, dk, dv]. Returns [T, H dv]."""
+    silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided, one dtype); state fp32 [slots, H, dk, dv]. Returns [T, H dv] as
+    `out_dtype` (default: that of the inputs)."""
+    dt = out_dtype or r.dtype
     if native_device(r) and RECURRENT_STEP and sm.max_q == 1 and r.shape[0] == sm.num_seqs:
-        return _recurrent_step(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
+        return _recurrent_step(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus, out_dtype=dt)
+    if dt != r.dtype:
+        r, k, v, g, z = (t.to(dt) for t in (r, k, v, g, z))
     if native_device(r) and CHUNK_RECURRENCE and r.dtype == torch.bfloat16 and dk == dv and dk in CHUNK_DK and dk != 96 \
             and all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (r, k, v, g, z)):
         return _chunk_recurrence(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
