@@ -6,7 +6,6 @@
 //   token_shift_mix  n mixes x_t + (x_(t-1) - x_t) mu_s of each row with the previous token's, as activation tensors
 //                    [n][T rounded up to whole tiles][W]; x_(-1) comes from the slot's carried row (zeros at a sequence's start), which takes the
 //                    portion's last row
-//   low_rank_decay   z = W2 tanh(W1 x) for steps of few rows, one workgroup per row, all fp32 between the weights
 //   time_mix_gates   r, k as fp32 and the decay f = exp(-exp(z + w0))
 //   recurrent_step   steps of single tokens, one workgroup per (sequence, head): rotation or decay, the state update
 //                      S <- diag(f) S + k v^T,   o = S^T q  (after the update)  or  o = (S_old + diag(u) k v^T)^T q,
@@ -108,61 +107,11 @@ __global__ __launch_bounds__(256) void time_mix_gates_kernel(const T* __restrict
   fo[i] = expf(-expf(ldf(z + t * ld_z + c) + w0[c]));
 }
 
-constexpr int kMaxRank = 256;
-
-template <typename T>
-__global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict__ x, int64_t ld_x, const T* __restrict__ w1,
-                                                             const T* __restrict__ w2, int W, int rank, int n,
-                                                             float* __restrict__ z) {
-  extern __shared__ float row[];   // [W]
-  __shared__ __attribute__((aligned(16))) float th[kMaxRank];
-  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int c = threadIdx.x; c < W; c += 256) row[c] = ldf(x + t * ld_x + c);
-  __syncthreads();
-  const bool quad = (W & 3) == 0;
-  for (int j0 = wave * 4; j0 < rank; j0 += 16) {   // four rows of W1 per wave at a time (past the last: it again, not stored)
-    float acc[4] = {0.f, 0.f, 0.f, 0.f};
-    if (quad) {
-      for (int c = 4 * lane; c < W; c += 256) {
-        float a[4], b[4][4];
-        ld4(row + c, a);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) ld4(w1 + (int64_t)min(j0 + j, rank - 1) * W + c, b[j]);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) acc[j] += a[0] * b[j][0] + a[1] * b[j][1] + a[2] * b[j][2] + a[3] * b[j][3];
-      }
-    } else {
-      for (int c = lane; c < W; c += 64)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) acc[j] += row[c] * ldf(w1 + (int64_t)min(j0 + j, rank - 1) * W + c);
-    }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      acc[j] = wave_sum(acc[j]);
-      if (lane == 0 && j0 + j < rank) th[j0 + j] = tanhf(acc[j]);
-    }
-  }
-  __syncthreads();
-  for (int c = threadIdx.x; c < n; c += 256) {
-    const T* wr = w2 + (int64_t)c * rank;
-    float acc = 0.f;
-    if ((rank & 3) == 0) {
-      for (int j = 0; j < rank; j += 4) {
-        float b[4];
-        ld4(wr + j, b);
-        acc += th[j] * b[0] + th[j + 1] * b[1] + th[j + 2] * b[2] + th[j + 3] * b[3];
-      }
-    } else {
-      for (int j = 0; j < rank; ++j) acc += th[j] * ldf(wr + j);
-    }
-    z[(int64_t)t * n + c] = acc;
-  }
-}
-
 // ------------------------------------------------------------------ single tokens
 struct StepArgs {
   const void *q, *k, *v, *g, *z;   // head h of token t at row t: columns h dk .. / h dv ..
   int64_t ld_q, ld_k, ld_v, ld_g, ld_z;
+  int z_f32;
   const float *decay, *w0, *bonus;   // decay [H]: retention; else w0 [H dk] beside z, bonus [H dk]
   const float* rot;
   int rot_rows, rot_dims;
@@ -212,7 +161,8 @@ __global__ __launch_bounds__(kStepThreads) void recurrent_step_kernel(const Step
       }
       k *= a.k_scale;
     } else {
-      f = expf(-expf(ldf((const T*)a.z + s * a.ld_z + h * dk + d) + a.w0[h * dk + d]));
+      const int64_t zi = s * a.ld_z + h * dk + d;
+      f = expf(-expf((a.z_f32 ? ((const float*)a.z)[zi] : bf2f(((const bf16*)a.z)[zi])) + a.w0[h * dk + d]));
       ruk = q * a.bonus[h * dk + d] * k;
     }
     qs[d] = q, ks[d] = k, fs[d] = f;
@@ -300,17 +250,8 @@ void time_mix_gates(const void* r, int64_t ld_r, const void* k, int64_t ld_k, co
                           (const T*)r, ld_r, (const T*)k, ld_k, (const T*)z, ld_z, w0, n, ro, fo, ko, total);)
 }
 
-int low_rank_decay(const void* x, int64_t ld_x, bool f32, const void* w1, const void* w2, int W, int rank, int n, float* z,
-                   int T_, hipStream_t st) {
-  if (T_ <= 0) return 0;
-  if (W < 1 || W > 16000 || rank < 1 || rank > kMaxRank || n < 1 || (uintptr_t)w1 % 16 || (uintptr_t)w2 % 16) return -1;
-  XGM_DISPATCH_T(f32, low_rank_decay_kernel<T><<<T_, 256, (size_t)W * sizeof(float), st>>>(
-                          (const T*)x, ld_x, (const T*)w1, (const T*)w2, W, rank, n, z);)
-  return 0;
-}
-
 int recurrent_step(const void* q, int64_t ld_q, const void* k, int64_t ld_k, const void* v, int64_t ld_v, const void* g,
-                   int64_t ld_g, const void* z, int64_t ld_z, bool f32, bool out_f32, const float* decay, const float* w0,
+                   int64_t ld_g, const void* z, int64_t ld_z, bool z_f32, bool f32, bool out_f32, const float* decay, const float* w0,
                    const float* bonus, const float* rot, int rot_rows, int rot_dims, float k_scale, const float* norm_w,
                    float eps, float* state, const int32_t* seq_lens, const int32_t* slots, const int32_t* positions,
                    void* out, int ns, int H, int dk, int dv, hipStream_t st) {
@@ -318,7 +259,7 @@ int recurrent_step(const void* q, int64_t ld_q, const void* k, int64_t ld_k, con
   if (H < 1 || dk < 1 || dk > kStepMaxDk || dv < 1 || dv > 8192 || (!decay && (!z || !w0 || !bonus)) || rot_dims % 2 ||
       rot_dims > dk || (rot_dims && !rot))
     return -1;
-  const StepArgs a = {q, k, v, g, z, ld_q, ld_k, ld_v, ld_g, ld_z, decay, w0, bonus, rot, rot_rows, rot_dims, k_scale,
+  const StepArgs a = {q, k, v, g, z, ld_q, ld_k, ld_v, ld_g, ld_z, z_f32, decay, w0, bonus, rot, rot_rows, rot_dims, k_scale,
                       norm_w, eps, state, seq_lens, slots, positions, out, H, dk, dv};
   const int cv = dv % 4 == 0 ? 4 : 1, ct = (dv + cv - 1) / cv, rg = ct < kStepThreads ? kStepThreads / ct : 1;
   const size_t lds = (size_t)rg * dv * sizeof(float);

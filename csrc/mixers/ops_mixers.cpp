@@ -71,12 +71,11 @@ void rotate_qk(const void*, bool, int64_t, int, int, int, int, const float*, int
                int, hipStream_t);
 void token_shift_mix(const float*, const float*, int, float*, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
                      void*, bool, int, int, int, hipStream_t);
-int low_rank_decay(const void*, int64_t, bool, const void*, const void*, int, int, int, float*, int, hipStream_t);
 void time_mix_gates(const void*, int64_t, const void*, int64_t, const void*, int64_t, bool, const float*, int, float*, float*,
                     float*, int, hipStream_t);
 int recurrent_step(const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
-                   int64_t, bool, bool, const float*, const float*, const float*, const float*, int, int, float, const float*,
-                   float, float*, const int32_t*, const int32_t*, const int32_t*, void*, int, int, int, int, hipStream_t);
+                   int64_t, bool, bool, bool, const float*, const float*, const float*, const float*, int, int, float,
+                   const float*, float, float*, const int32_t*, const int32_t*, const int32_t*, void*, int, int, int, int, hipStream_t);
 void decay_gates(const void*, bool, int64_t, int, int, int, float, const void*, int64_t, const float*, float, float*, float*,
                  float*, int, hipStream_t);
 void moe_combine(const float*, const int32_t*, const float*, int, int, int, float*, hipStream_t);
@@ -391,13 +390,6 @@ PYBIND11_MODULE(_mixers, m) {
                          T, pitch, W, S(st));
     check(0, "token_shift_mix");
   });
-  m.def("low_rank_decay", [](uintptr_t x, int64_t ld_x, bool f32, uintptr_t w1, uintptr_t w2, int W, int rank, int n,
-                             uintptr_t z, int T, uintptr_t st) {
-    if (ld_x < W) throw std::invalid_argument("low_rank_decay: row stride below the width");
-    int rc = xgm::low_rank_decay(P<const void>(x), ld_x, f32, P<const void>(w1), P<const void>(w2), W, rank, n, P<float>(z),
-                                 T, S(st));
-    check(rc, "low_rank_decay");
-  });
   m.def("time_mix_gates", [](uintptr_t r, int64_t ld_r, uintptr_t k, int64_t ld_k, uintptr_t z, int64_t ld_z, bool f32,
                              uintptr_t w0, int n, uintptr_t ro, uintptr_t fo, uintptr_t ko, int T, uintptr_t st) {
     if (n < 1 || ld_r < n || ld_k < n || ld_z < n) throw std::invalid_argument("time_mix_gates: inconsistent sizes");
@@ -406,7 +398,7 @@ PYBIND11_MODULE(_mixers, m) {
     check(0, "time_mix_gates");
   });
   m.def("recurrent_step", [](uintptr_t q, int64_t ld_q, uintptr_t k, int64_t ld_k, uintptr_t v, int64_t ld_v, uintptr_t g,
-                             int64_t ld_g, uintptr_t z, int64_t ld_z, bool f32, bool out_f32, uintptr_t decay,
+                             int64_t ld_g, uintptr_t z, int64_t ld_z, bool z_f32, bool f32, bool out_f32, uintptr_t decay,
                              uintptr_t w0, uintptr_t bonus, uintptr_t rot, int rot_rows, int rot_dims, float k_scale, uintptr_t norm_w,
                              float eps, uintptr_t state, uintptr_t sl, uintptr_t slots, uintptr_t pos, uintptr_t out, int ns,
                              int H, int dk, int dv, uintptr_t st) {
@@ -414,7 +406,7 @@ PYBIND11_MODULE(_mixers, m) {
     if (ld_q < nk || ld_k < nk || ld_v < nv || ld_g < nv || (z && ld_z < nk) || rot_dims < 0 || (rot_dims && rot_rows < 1))
       throw std::invalid_argument("recurrent_step: inconsistent sizes");
     int rc = xgm::recurrent_step(P<const void>(q), ld_q, P<const void>(k), ld_k, P<const void>(v), ld_v, P<const void>(g),
-                                 ld_g, P<const void>(z), ld_z, f32, out_f32, P<const float>(decay), P<const float>(w0),
+                                 ld_g, P<const void>(z), ld_z, z_f32, f32, out_f32, P<const float>(decay), P<const float>(w0),
                                  P<const float>(bonus), P<const float>(rot), rot_rows, rot_dims, k_scale,
                                  P<const float>(norm_w), eps, P<float>(state), P<const int32_t>(sl), P<const int32_t>(slots),
                                  P<const int32_t>(pos), P<void>(out), ns, H, dk, dv, S(st));

@@ -641,20 +641,6 @@ def test_stacked_products_of_short_steps(T, G, K, N):
     assert y.shape == (G, R, N) and float((y[:, :T].cpu().to(F64) - ref[:, :T]).abs().max()) < 1e-4 * float(ref.abs().max())
 
 
-@pytest.mark.parametrize("device,dtype", CASES)
-@pytest.mark.parametrize("T,W,rank,n", [(1, 50, 1, 16), (7, 64, 6, 60), (64, 130, 16, 40), (64, 512, 64, 256), (5, 33, 130, 300),
-                                        (90, 64, 8, 64)])
-def test_low_rank_decay(device, dtype, T, W, rank, n):
-    dt = getattr(torch, dtype)
-    g = torch.Generator().manual_seed(T + W)
-    wide = bf(torch.randn(T, W + 6, generator=g))
-    w1, w2 = bf(torch.randn(rank, W, generator=g) / W ** 0.5), bf(torch.randn(n, rank, generator=g) / rank ** 0.5)
-    d = lambda t: t.to(dt).to(device)  # noqa: E731
-    z = sq.low_rank_decay(d(wide)[:, :W], d(w1), d(w2))
-    ref = torch.tanh(wide[:, :W] @ w1.T) @ w2.T
-    assert float((z.cpu().to(F64) - ref).abs().max()) < (1e-5 if dtype == "float32" else 3e-2) * float(ref.abs().max())
-
-
 @pytest.mark.parametrize("device", OP_CASES)
 @pytest.mark.parametrize("T,E,top,W", [(9, 1, 1, 32), (9, 5, 2, 50), (40, 8, 8, 64), (300, 12, 3, 64), (5, 100, 70, 33),
                                        (20, 16, 4, 4096)])

@@ -109,8 +109,8 @@ class TimeMix(nn.Module):
             r, k, v, g = sq.stacked_linear(mixed[:4], self.rkvg, T)[:, :T].unbind(0)
         else:
             r, k, v, g = (F.linear(mixed[j], self.rkvg[j]) for j in range(4))
-        z = sq.low_rank_decay(mixed[4][:T], self.w1, self.w2)
-        y = sq.time_mix(r, k, v, g, z.to(r.dtype), self.w0, self.u, self.norm, self.eps, self.H, self.dk, self.dk, lc.gla, sm,
+        z = F.linear(sq.tanh_cols(F.linear(mixed[4][:T], self.w1), 0, self.rank), self.w2)
+        y = sq.time_mix(r, k, v, g, z, self.w0, self.u, self.norm, self.eps, self.H, self.dk, self.dk, lc.gla, sm,
                         dtype)
         return F.linear(y, self.o)
 

@@ -1385,13 +1385,16 @@ def token_shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, sm: 
     return out
 
 
-STACKED_MAX_ROWS = 64   # steps of up to this many rows run products with inputs of their own as one launch
+STACKED_MAX_ROWS = 64         # steps of up to this many rows run products with inputs of their own as one launch ...
+STACKED_MAX_ELEMS = 1 << 23   # ... for weights up to this size (measured on 64 rows, four products: 21 us against 47 us for
+                              # 2048 x 2048 weights, 68 us against 60 us for 4096 x 4096)
 _STACKED_LAYOUT = {}
 
 
 def stacked_tile(T: int, K: int, N: int, w: torch.Tensor) -> int:
     """Rows per tile of stacked_linear for steps of T rows, 0 where separate matrix products are used."""
-    if not (native_device(w) and MOE_MFMA and w.dtype == torch.bfloat16 and T <= STACKED_MAX_ROWS and K % 32 == 0 and N % 16 == 0):
+    if not (native_device(w) and MOE_MFMA and w.dtype == torch.bfloat16 and T <= STACKED_MAX_ROWS and K % 32 == 0 and N % 16 == 0
+            and K * N <= STACKED_MAX_ELEMS):
         return 0
     return 16 if T <= 16 else 32
 
@@ -1415,23 +1418,6 @@ def stacked_linear(x: torch.Tensor, w: torch.Tensor, T: int) -> torch.Tensor:
     return y
 
 
-LOW_RANK_MAX_ROWS, LOW_RANK_MAX = 64, 256   # steps and ranks of the one-launch form
-
-
-def low_rank_decay(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor) -> torch.Tensor:
-    """w2 tanh(w1 x): x [T, W] row-strided activations, w1 [rank, W], w2 [n, rank]. Short steps on the GPU: one launch, fp32
-    [T, n]; else two matrix products, in the activation dtype."""
-    T, W = x.shape
-    rank, n = w1.shape[0], w2.shape[0]
-    if native_device(x) and T <= LOW_RANK_MAX_ROWS and rank <= LOW_RANK_MAX:
-        assert x.stride(1) == 1 and x.dtype == w1.dtype == w2.dtype and w1.is_contiguous() and w2.is_contiguous()
-        z = torch.empty(T, n, dtype=torch.float32, device=x.device)
-        mixers().low_rank_decay(x.data_ptr(), x.stride(0), is_f32(x), w1.data_ptr(), w2.data_ptr(), W, rank, n, z.data_ptr(),
-                                T, stream_ptr())
-        return z
-    return torch.nn.functional.linear(tanh_cols(torch.nn.functional.linear(x, w1), 0, rank), w2)
-
-
 def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.Tensor):
     """(r, exp(-exp(z + w0)), k) as fp32 [T, n]: the inputs of gated_linear_scan with a data-dependent decay per key
     channel. r, k, z row-strided activation tensors; w0 fp32 [n]."""
@@ -1449,11 +1435,12 @@ def time_mix_gates(r: torch.Tensor, k: torch.Tensor, z: torch.Tensor, w0: torch.
 def _recurrent_step(q, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, decay=None, w0=None, bonus=None, rot=None, rot_dims=0,
                     k_scale=1.0, out_dtype=None):
     """A step of single tokens: recurrence, per-head norm and gate in one kernel. Returns [T, H dv]."""
-    assert all(t.stride(1) == 1 and t.dtype == q.dtype for t in (q, k, v, g)) and (z is None or (z.stride(1) == 1 and z.dtype == q.dtype))
+    assert all(t.stride(1) == 1 and t.dtype == q.dtype for t in (q, k, v, g)) and (z is None or z.stride(1) == 1)
     assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, dk, dv)
     out = torch.empty(q.shape[0], H * dv, dtype=out_dtype or q.dtype, device=q.device)
     mixers().recurrent_step(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), g.data_ptr(),
-                            g.stride(0), _p(z), z.stride(0) if z is not None else 0, is_f32(q), is_f32(out), _p(decay), _p(w0),
+                            g.stride(0), _p(z), z.stride(0) if z is not None else 0,
+                            is_f32(z) if z is not None else False, is_f32(q), is_f32(out), _p(decay), _p(w0),
                             _p(bonus), _p(rot) if rot_dims else 0, rot.shape[0] if rot_dims else 0, rot_dims, float(k_scale), _p(norm_w),
                             float(eps), state.data_ptr(), _i32(sm.seq_lens).data_ptr(), _i32(sm.slots).data_ptr(),
                             _i32(sm.positions).data_ptr(), out.data_ptr(), q.shape[0], H, dk, dv, stream_ptr())
@@ -1535,13 +1522,12 @@ def time_mix(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor,
              sm: SeqMeta, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
     """Per head, with the decay w = exp(-exp(z + w0)) per key channel: o = (S + diag(u) k v^T)^T r with the bonus u for the
     current token, then S <- diag(w) S + k v^T; each head's o divided by its own root mean square, times norm_w, times
-    silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided, one dtype); state fp32 [slots, H, dk, dv]. Returns [T, H dv] as
+    silu(g). r, k, z [T, H dk], v, g [T, H dv] (row-strided; r, k, v, g of one dtype); state fp32 [slots, H, dk, dv]. Returns [T, H dv] as
     `out_dtype` (default: that of the inputs)."""
     dt = out_dtype or r.dtype
     if native_device(r) and RECURRENT_STEP and sm.max_q == 1 and r.shape[0] == sm.num_seqs:
         return _recurrent_step(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus, out_dtype=dt)
-    if dt != r.dtype:
-        r, k, v, g, z = (t.to(dt) for t in (r, k, v, g, z))
+    r, k, v, g, z = (t.to(dt) for t in (r, k, v, g, z))
     if native_device(r) and CHUNK_RECURRENCE and r.dtype == torch.bfloat16 and dk == dv and dk in CHUNK_DK and dk != 96 \
             and all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (r, k, v, g, z)):
         return _chunk_recurrence(r, k, v, g, z, H, dk, dv, state, sm, norm_w, eps, w0=w0, bonus=bonus)
