@@ -533,7 +533,7 @@ __global__ __launch_bounds__(256) void head_norm_rope_cache_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ slot_mapping, TO* __restrict__ q_out,
     TO* __restrict__ kcache, TO* __restrict__ vcache, int whole, int half, const TI* __restrict__ v_first,
     int64_t ld_vf, const float* __restrict__ v_mix, int vec) {
-  __shared__ float red[4];
+  __shared__ float red[8];
   const int t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const TI* row = src + (int64_t)t * ld;
@@ -542,23 +542,31 @@ __global__ __launch_bounds__(256) void head_norm_rope_cache_kernel(
   const float* cs = nullptr;
   if (rot && rot_dims > 0) cs = rot + (int64_t)min(max(positions[t], 0), rot_rows - 1) * rot_dims;  // [rot_dims / 2][2]
   float rq = 1.f, rk = 1.f;
-  if (whole) {
-    if (wq) {
-      float ss = 0.f;
-      for (int c = threadIdx.x; c < nq; c += blockDim.x) {
+  if (whole && (wq || wk)) {   // both vectors' statistics in one pass over [q | k] and one exchange between the waves
+    float sq = 0.f, sk = 0.f;
+    if (vec) {
+      for (int c = 4 * threadIdx.x; c < nq + nk; c += 4 * blockDim.x) {
+        float a[4];
+        ld4(row + c, a);
+        const float ss = a[0] * a[0] + a[1] * a[1] + a[2] * a[2] + a[3] * a[3];
+        if (c < nq) sq += ss;
+        else sk += ss;
+      }
+    } else {
+      for (int c = threadIdx.x; c < nq + nk; c += blockDim.x) {
         const float a = ldf(row + c);
-        ss += a * a;
+        if (c < nq) sq += a * a;
+        else sk += a * a;
       }
-      rq = 1.f / sqrtf(block_sum(ss, red) / (float)nq + eps);
     }
-    if (wk) {
-      float ss = 0.f;
-      for (int c = threadIdx.x; c < nk; c += blockDim.x) {
-        const float a = ldf(row + nq + c);
-        ss += a * a;
-      }
-      rk = 1.f / sqrtf(block_sum(ss, red) / (float)nk + eps);
-    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if (lane == 0) red[wave] = sq, red[4 + wave] = sk;
+    __syncthreads();
+    sq = sk = 0.f;
+    for (int i = 0; i < nw; ++i) sq += red[i], sk += red[4 + i];
+    if (wq) rq = 1.f / sqrtf(sq / (float)nq + eps);
+    if (wk) rk = 1.f / sqrtf(sk / (float)nk + eps);
   }
   const int hr = rot_dims / 2;
   if (vec) {
