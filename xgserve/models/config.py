@@ -492,6 +492,8 @@ def _taritar_tiny_layers():
 
 register(taritar_config("taritar-tiny", 128, 512, _taritar_tiny_layers(), streams=3, embed_scale=2.0, logit_softcap=25.0,
                         max_position=1024))
+
+
 def bazurax_config(name: str, width: int, vocab: int, layers: List[dict], eps: float = 1e-6,
                    max_position: int = 131072) -> ModelConfig:
     """A Bazurax model: layers x <- x + L(mixer(x)), x <- x + L(ff(x)) with a layer norm L on each sublayer's output and on
